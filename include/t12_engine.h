@@ -32,7 +32,9 @@ void* t12_engine_create_synthetic(int n_vocab, int n_embd, int n_head, int n_hea
 /* create_synthetic_gamilorn: the same for a model of the Gamilorn family; config_json is the text of a config.json, rank
  * the width of the decay projection (a checkpoint's tensor gives it otherwise). */
 void* t12_engine_create_synthetic_gamilorn(const char* config_json, int rank, uint64_t seed, float p_outlier);
-const char* t12_engine_family(void* model);                          /* model_family: "llama", "gamilorn" */
+/* create_synthetic_davasun: the same for a model of the Davasun family. */
+void* t12_engine_create_synthetic_davasun(const char* config_json, uint64_t seed, float p_outlier);
+const char* t12_engine_family(void* model);                          /* model_family: "llama", "gamilorn", "davasun" */
 int   t12_engine_vocab(void* model);                                 /* Model::config.n_vocab */
 int   t12_engine_save(void* model, const char* dir);                 /* save_model: the files of convert_model.py:127-152; 0 = ok */
 void  t12_engine_free_model(void* model);                            /* free_model */

@@ -101,7 +101,7 @@ Model* load_model(const std::string& model_path, int device_id = 0);
 // loading, or the split-12 directory save_model writes for it -- is checked and loaded by that family.
 bool check_model_dir(const std::string& model_path, std::string& err);
 void free_model(Model* model);
-const char* model_family(const Model* model);    // "llama", "gamilorn"
+const char* model_family(const Model* model);    // "llama", "gamilorn", "davasun"
 
 // ---- not in the reference -----------------------------------------------------
 // A random-init model of the given shape generated and packed ON THE GPU:
@@ -111,6 +111,8 @@ Model* create_synthetic_model(const ModelConfig& cfg, uint64_t seed, int max_seq
 // The same for a model of the Gamilorn family: config_json is the text of a config.json, rank the width of the decay
 // projection (a checkpoint's tensor gives it otherwise).
 Model* create_synthetic_gamilorn(const std::string& config_json, int rank, uint64_t seed, float p_outlier = 3e-4f);
+// The same for a model of the Davasun family.
+Model* create_synthetic_davasun(const std::string& config_json, uint64_t seed, float p_outlier = 3e-4f);
 // Writes the model in the directory layout load_model reads (for the Llama family the files
 // engine/convert_model.py:57-62,127-152 emits).
 bool save_model(const Model* model, const std::string& dir);

@@ -26,7 +26,7 @@ def build(tmp, with_model_dir):
         # model.cpp also holds the GPU half of the loader: its HIP and library calls resolve against the built
         # libraries, none of them runs (check_model_dir is host code only)
         cmd += ["-DWITH_MODEL_DIR", "-D__HIP_PLATFORM_AMD__", "-I/opt/rocm/include", "-I" + os.path.join(ROOT, "turbo-lossless_amd", "csrc"),
-                os.path.join(ENG, "model.cpp"), os.path.join(ENG, "gamilorn_model.cpp"), os.path.join(ENG, "checkpoint.cpp"), "-L" + os.path.join(ROOT, "turbo-lossless_amd"), "-lturbo12",
+                os.path.join(ENG, "model.cpp"), os.path.join(ENG, "gamilorn_model.cpp"), os.path.join(ENG, "davasun_model.cpp"), os.path.join(ENG, "part_store.cpp"), os.path.join(ENG, "checkpoint.cpp"), "-L" + os.path.join(ROOT, "turbo-lossless_amd"), "-lturbo12",
                 "-L/opt/rocm/lib", "-lamdhip64", "-Wl,-rpath," + os.path.join(ROOT, "turbo-lossless_amd"), "-Wl,-rpath,/opt/rocm/lib"]
     r = subprocess.run(cmd + ["-o", exe], capture_output=True, text=True)
     assert r.returncode == 0, r.stderr[-3000:]

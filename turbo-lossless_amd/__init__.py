@@ -123,6 +123,7 @@ _SIGS = {
     "t12_engine_family": (C.c_char_p, [_vp]),
     "t12_engine_vocab": (_i, [_vp]),
     "t12_engine_create_synthetic_gamilorn": (_vp, [C.c_char_p, _i, C.c_uint64, C.c_float]),
+    "t12_engine_create_synthetic_davasun": (_vp, [C.c_char_p, C.c_uint64, C.c_float]),
     "t12_engine_create_state_with": (_vp, [_vp, _i, _i, _i, _i, _i]),
     "t12_engine_prefill_logits": (_i, [_vp, _i, C.POINTER(_i), _i, C.POINTER(_i), _i, _i, _vp]),
     "t12_engine_load": (_vp, [C.c_char_p, _i]),
@@ -410,6 +411,13 @@ class Engine:
         """A random-init model of the Gamilorn family; config: the dict config.json would hold."""
         import json
         h = lib.t12_engine_create_synthetic_gamilorn(json.dumps(config).encode(), int(rank), seed, p_outlier)
+        return cls(h, batch, per_sequence, prompt_rows, fp32)
+
+    @classmethod
+    def synthetic_davasun(cls, config, seed=4000, batch=1, p_outlier=3e-4, per_sequence=0, prompt_rows=0, fp32=False):
+        """A random-init model of the Davasun family; config: the dict config.json would hold."""
+        import json
+        h = lib.t12_engine_create_synthetic_davasun(json.dumps(config).encode(), seed, p_outlier)
         return cls(h, batch, per_sequence, prompt_rows, fp32)
 
     @property

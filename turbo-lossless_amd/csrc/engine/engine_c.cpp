@@ -69,6 +69,11 @@ void* t12_engine_create_synthetic_gamilorn(const char* config_json, int rank, ui
     return guarded_ptr([&]() -> void* { return create_synthetic_gamilorn(config_json ? config_json : "", rank, seed, p_outlier); });
 }
 
+void* t12_engine_create_synthetic_davasun(const char* config_json, uint64_t seed, float p_outlier)
+{
+    return guarded_ptr([&]() -> void* { return create_synthetic_davasun(config_json ? config_json : "", seed, p_outlier); });
+}
+
 const char* t12_engine_family(void* model) { return model_family((const Model*)model); }
 int t12_engine_vocab(void* model) { return ((const Model*)model)->config.n_vocab; }
 

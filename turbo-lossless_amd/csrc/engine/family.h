@@ -67,8 +67,8 @@ struct ModelFamily {
 };
 
 // (not const: hipcc would make constant-initialised host tables part of the device code as well)
-extern ModelFamily kLlamaFamily, kGamilornFamily;
-extern FamilyRun kLlamaRun, kGamilornRun;
+extern ModelFamily kLlamaFamily, kGamilornFamily, kDavasunFamily;
+extern FamilyRun kLlamaRun, kGamilornRun, kDavasunRun;
 
 const ModelFamily& family_of(const Model* m);
 

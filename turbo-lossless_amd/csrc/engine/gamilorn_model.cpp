@@ -1,28 +1,22 @@
 // Configuration, loading and saving of Gamilorn models (gamilorn.h).
-//
-// Two directory forms, both with the model's config.json:
-//   * a checkpoint, config.json + model.safetensors: the tensors are fused and packed to split-12 on the GPU while they
-//     are loaded;
-//   * what save_model writes: the packed tensors as the seven files every split-12 tensor of this build has, fp32
-//     vectors as <name>.f32.bin, bf16 tables as <name>.bf16.bin.
+// Directory forms: part_store.h.
 #include "gamilorn.h"
 
 #include <cmath>
 #include <cstdio>
 #include <cstdlib>
 #include <cstring>
-#include <functional>
 
-#include "checkpoint.h"
 #include "family.h"
 #include "json.h"
-#include "model_store.h"
-#include "t12_abi.h"
-
-extern "C" int t12_synth_normal_bf16(void*, size_t, uint64_t, float, float, float, void*);
-extern "C" int t12_fill_f32(void*, size_t, float, void*);
+#include "part_store.h"
 
 using namespace model_store;
+using part_store::Parts;
+using part_store::ends_with;
+using part_store::is_checkpoint;
+using part_store::layer_name;
+using part_store::values;
 
 namespace gamilorn {
 
@@ -31,14 +25,6 @@ Data* data_of(const Model* m) { return (Data*)m->family_data; }
 namespace {
 
 const char* const kArchitecture = "Gamilorn";
-
-bool read_text(const std::string& path, std::string& text)
-{
-    std::vector<uint8_t> b;
-    if (!read_file(path, b, true)) return false;
-    text.assign((const char*)b.data(), b.size());
-    return true;
-}
 
 // Everything config.json says.  The rank of the decay projection and the position table's length are sizes of tensors.
 void parse_config(const std::string& text, Config& c)
@@ -81,16 +67,7 @@ void parse_config(const std::string& text, Config& c)
     }
 }
 
-std::string layer_name(size_t i, const char* what) { return "l" + std::to_string(i) + "." + what; }
-
-// ---- the parts a model is stored and held as.  One walk serves checking, loading, saving and freeing.
-struct Parts {
-    // fused or single matrix [M, K]
-    std::function<void(const std::string&, CompressedWeight&, int M, int K)> weight;
-    std::function<void(const std::string&, float*&, size_t n)> vector;
-    std::function<void(const std::string&, int16_t*&, size_t n)> table;
-};
-
+// ---- the parts a model is stored and held as
 void walk(const Config& c, Model* m, Data* d, const Parts& p)
 {
     p.table("embed", m->token_embd, (size_t)c.vocab * c.width);
@@ -181,157 +158,72 @@ bool open_checkpoint(const std::string& dir, Config& c, Checkpoint& ck, std::str
     return true;
 }
 
-float bf16_value(const uint8_t* p)
-{
-    uint16_t b;
-    memcpy(&b, p, 2);
-    const uint32_t u = (uint32_t)b << 16;
-    float f;
-    memcpy(&f, &u, 4);
-    return f;
-}
-
 void load_checkpoint(const Checkpoint& ck, const Config& c, Model* m, Data* d)
 {
-    auto bytes = [&](const std::string& name) { return ck.data(*ck.find(name)); };
-    auto count = [&](const std::string& name) { return (size_t)ck.find(name)->count(); };
-    auto values = [&](const std::string& name, float add) {
-        std::vector<float> v(count(name));
-        const uint8_t* b = bytes(name);
-        for (size_t i = 0; i < v.size(); i++) v[i] = bf16_value(b + 2 * i) + add;
-        return v;
-    };
-    // matrices next to each other along K (one entry: the matrix itself), or below each other
-    auto beside = [&](const std::vector<std::string>& names, int M, std::vector<uint8_t>& out) {
-        for (int r = 0; r < M; r++)
-            for (const std::string& n : names) {
-                const size_t row = count(n) / M * 2;
-                const uint8_t* b = bytes(n) + row * r;
-                out.insert(out.end(), b, b + row);
-            }
-    };
-    auto below = [&](const std::vector<std::string>& names, std::vector<uint8_t>& out) {
-        for (const std::string& n : names) out.insert(out.end(), bytes(n), bytes(n) + count(n) * 2);
-    };
-    auto ends = [](const std::string& s, const char* e) {
-        const size_t n = strlen(e);
-        return s.size() >= n && s.compare(s.size() - n, n, e) == 0;
-    };
     Parts p;
-    p.table = [&](const std::string& name, int16_t*& dst, size_t n) { dst = upload<int16_t>(bytes(name), n); };
+    p.table = [&](const std::string& name, int16_t*& dst, size_t n) { dst = upload<int16_t>(ck.data(*ck.find(name)), n); };
     p.vector = [&](const std::string& name, float*& dst, size_t n) {
         const std::string base = name.substr(0, name.find('.') + 1);
         std::vector<float> v;
-        if (ends(name, "norm1") || ends(name, "norm2") || name == "final.norm") v = values(name, 1.0f);   // stored around zero
-        else if (ends(name, "mix.in.b")) {
+        if (ends_with(name, "norm1") || ends_with(name, "norm2") || name == "final.norm") v = values(ck, name, 1.0f);   // stored around zero
+        else if (ends_with(name, "mix.in.b")) {
             v.assign(n, 0.0f);
             const LayerConfig& k = d->layers[std::stoul(name.substr(1))].c;
             auto put = [&](const char* t, int off) {
-                const std::vector<float> b = values(base + t, 0.0f);
+                const std::vector<float> b = values(ck, base + t);
                 std::copy(b.begin(), b.end(), v.begin() + off);
             };
             put("mix.left.q.b", k.q_off());
             put("mix.left.k.b", k.k_off());
             put("mix.left.v.b", k.v_off());
             put("mix.right.a.b", k.a_off());
-        } else if (ends(name, "mix.head_bias")) v = values(base + "mix.left.pb", 0.0f);
-        else if (ends(name, "mix.w2t")) {
-            const std::vector<float> w = values(base + "mix.right.w2", 0.0f);
+        } else if (ends_with(name, "mix.head_bias")) v = values(ck, base + "mix.left.pb");
+        else if (ends_with(name, "mix.w2t")) {
+            const std::vector<float> w = values(ck, base + "mix.right.w2");
             const LayerConfig& k = d->layers[std::stoul(name.substr(1))].c;
             v.resize(n);
             for (int r = 0; r < k.rank; r++)
                 for (int i = 0; i < k.del(); i++) v[(size_t)r * k.del() + i] = w[(size_t)i * k.rank + r];
-        } else if (ends(name, "mix.w0")) v = values(base + "mix.right.w0", 0.0f);
-        else if (ends(name, "mix.norm")) v = values(base + "mix.right.norm", 0.0f);
-        else v = values(name, 0.0f);
+        } else if (ends_with(name, "mix.w0")) v = values(ck, base + "mix.right.w0");
+        else if (ends_with(name, "mix.norm")) v = values(ck, base + "mix.right.norm");
+        else v = values(ck, name);
         dst = upload<float>(v.data(), n);
     };
     p.weight = [&](const std::string& name, CompressedWeight& w, int M, int K) {
         const std::string b = name.substr(0, name.find('.') + 1);
-        std::vector<uint8_t> bits;
-        bits.reserve((size_t)M * K * 2);
-        if (ends(name, "mix.in"))
-            below({b + "mix.left.q", b + "mix.left.k", b + "mix.left.v", b + "mix.right.r", b + "mix.right.k", b + "mix.right.v",
-                   b + "mix.right.a", b + "mix.right.g", b + "mix.right.w1"}, bits);
-        else if (ends(name, "mix.out")) beside({b + "mix.left.o", b + "mix.right.o"}, M, bits);
-        else below({name}, bits);
-        uint16_t* dev = upload<uint16_t>(bits.data(), (size_t)M * K);
-        const bool ok = pack_on_gpu(dev, M, K, w);
-        (void)hipFree(dev);
-        if (!ok) engine_fail("packing %s (%d x %d) failed: %s", name.c_str(), M, K, t12_last_error());
+        if (ends_with(name, "mix.in"))
+            part_store::pack(name, part_store::below(ck, {b + "mix.left.q", b + "mix.left.k", b + "mix.left.v", b + "mix.right.r", b + "mix.right.k",
+                                                          b + "mix.right.v", b + "mix.right.a", b + "mix.right.g", b + "mix.right.w1"}), M, K, w);
+        else if (ends_with(name, "mix.out")) part_store::pack(name, part_store::beside(ck, {b + "mix.left.o", b + "mix.right.o"}, M), M, K, w);
+        else part_store::pack(name, part_store::below(ck, {name}), M, K, w);
     };
     walk(c, m, d, p);
 }
 
 // ---- the packed directory ----------------------------------------------------------------------------------------
-std::string vec_file(const std::string& dir, const std::string& n) { return dir + "/" + n + ".f32.bin"; }
-std::string table_file(const std::string& dir, const std::string& n) { return dir + "/" + n + ".bf16.bin"; }
-
 bool check_packed(const std::string& dir, Config& c, std::string& err)
 {
-    const long long pos = file_size(table_file(dir, "pos"));
+    const long long pos = file_size(part_store::table_file(dir, "pos"));
     if (pos <= 0 || pos % (2LL * c.width)) return fail(err, "neither model.safetensors nor a usable pos.bf16.bin in " + dir);
     c.max_positions = (int)(pos / (2LL * c.width));
     for (size_t i = 0; i < c.layers.size(); i++) {
-        const long long b = file_size(vec_file(dir, layer_name(i, "mix.w2t"))), per = 4LL * c.layers[i].del();
+        const long long b = file_size(part_store::vector_file(dir, layer_name(i, "mix.w2t"))), per = 4LL * c.layers[i].del();
         if (b <= 0 || b % per || b / per > 512) return fail(err, layer_name(i, "mix.w2t") + " is missing or has the wrong size");
         c.layers[i].rank = (int)(b / per);
     }
     Model m;
     Data d;
     empty_layers(c, d);
-    bool ok = true;
-    Parts p;
-    p.weight = [&](const std::string& n, CompressedWeight&, int M, int K) { ok = ok && check_tensor(dir, n, M, K, err); };
-    p.vector = [&](const std::string& n, float*&, size_t k) {
-        if (ok && file_size(vec_file(dir, n)) != (long long)k * 4) ok = fail(err, n + ".f32.bin missing or not the right size");
-    };
-    p.table = [&](const std::string& n, int16_t*&, size_t k) {
-        if (ok && file_size(table_file(dir, n)) != (long long)k * 2) ok = fail(err, n + ".bf16.bin missing or not the right size");
-    };
-    walk(c, &m, &d, p);
-    return ok;
-}
-
-bool load_packed(const std::string& dir, const Config& c, Model* m, Data* d)
-{
-    bool ok = true;
-    Parts p;
-    p.weight = [&](const std::string& n, CompressedWeight& w, int, int) { ok = ok && load_compressed(dir, n, w); };
-    auto bytes = [&](const std::string& path, size_t want) {
-        std::vector<uint8_t> b;
-        if (!read_file(path, b) || b.size() != want) ok = false;
-        return b;
-    };
-    p.vector = [&](const std::string& n, float*& v, size_t k) {
-        const std::vector<uint8_t> b = bytes(vec_file(dir, n), k * 4);
-        if (ok) v = upload<float>(b.data(), k);
-    };
-    p.table = [&](const std::string& n, int16_t*& v, size_t k) {
-        const std::vector<uint8_t> b = bytes(table_file(dir, n), k * 2);
-        if (ok) v = upload<int16_t>(b.data(), k);
-    };
-    walk(c, m, d, p);
-    return ok;
+    return part_store::check_packed(dir, [&](const Parts& p) { walk(c, &m, &d, p); }, err);
 }
 
 // ---- family entries ------------------------------------------------------------------------------------------------
-bool owns(const std::string& dir)
-{
-    std::string text;
-    if (!read_text(dir + "/config.json", text)) return false;
-    try {
-        const Json j = Json::parse(text);
-        return j.has("architecture") && j.at("architecture").kind == Json::STR && j.at("architecture").text == kArchitecture;
-    } catch (const JsonError&) {
-        return false;
-    }
-}
+bool owns(const std::string& dir) { return part_store::has_architecture(dir, kArchitecture); }
 
 bool read_config(const std::string& dir, Config& c, std::string& err)
 {
     std::string text;
-    if (!read_text(dir + "/config.json", text)) return fail(err, "no config.json in " + dir);
+    if (!part_store::read_config_text(dir, text)) return fail(err, "no config.json in " + dir);
     try {
         parse_config(text, c);
     } catch (const JsonError& e) {
@@ -339,8 +231,6 @@ bool read_config(const std::string& dir, Config& c, std::string& err)
     }
     return true;
 }
-
-bool is_checkpoint(const std::string& dir) { return file_size(dir + "/model.safetensors") >= 0; }
 
 bool check(const std::string& dir, std::string& err)
 {
@@ -354,11 +244,7 @@ bool check(const std::string& dir, std::string& err)
 void release(Model* m)
 {
     Data* d = data_of(m);
-    Parts p;
-    p.weight = [](const std::string&, CompressedWeight& w, int, int) { free_weight(w); };
-    p.vector = [](const std::string&, float*& v, size_t) { if (v) (void)hipFree(v); v = nullptr; };
-    p.table = [](const std::string&, int16_t*& v, size_t) { if (v) (void)hipFree(v); v = nullptr; };
-    walk(d->config, m, d, p);
+    part_store::release([&](const Parts& p) { walk(d->config, m, d, p); });
     delete d;
     delete m;
 }
@@ -419,7 +305,7 @@ Model* load(const std::string& dir)
     Model* m = new_model(c);
     try {
         if (raw) load_checkpoint(ck, c, m, data_of(m));
-        else if (!load_packed(dir, c, m, data_of(m))) {
+        else if (!part_store::load_packed(dir, [&](const Parts& p) { walk(c, m, data_of(m), p); })) {
             release(m);
             return nullptr;
         }
@@ -436,21 +322,7 @@ bool save(const Model* cm, const std::string& dir)
 {
     Model* m = const_cast<Model*>(cm);                     // the walk hands out references; nothing is changed
     Data* d = data_of(m);
-    {
-        std::ofstream f(dir + "/config.json", std::ios::binary);
-        f.write(d->config.text.data(), (std::streamsize)d->config.text.size());
-        if (!f) {
-            fprintf(stderr, "Cannot write: %s/config.json (the directory must exist)\n", dir.c_str());
-            return false;
-        }
-    }
-    bool ok = true;
-    Parts p;
-    p.weight = [&](const std::string& n, CompressedWeight& w, int, int) { ok = ok && save_weight(dir, n, w); };
-    p.vector = [&](const std::string& n, float*& v, size_t k) { ok = ok && dump<float>(vec_file(dir, n), v, k); };
-    p.table = [&](const std::string& n, int16_t*& v, size_t k) { ok = ok && dump<int16_t>(table_file(dir, n), v, k); };
-    walk(d->config, m, d, p);
-    return ok;
+    return part_store::save_packed(dir, d->config.text, [&](const Parts& p) { walk(d->config, m, d, p); });
 }
 
 }  // namespace
@@ -478,30 +350,14 @@ Model* create_synthetic_gamilorn(const std::string& config_json, int rank, uint6
     }
     for (LayerConfig& k : c.layers) k.rank = rank;
     Model* m = new_model(c);
-    uint64_t s = seed;
-    Parts p;
-    p.weight = [&](const std::string& n, CompressedWeight& w, int M, int K) {
-        uint16_t* stage = device_alloc<uint16_t>((size_t)M * K);
-        const bool ok = t12_synth_normal_bf16(stage, (size_t)M * K, ++s, 0.02f, p_outlier, 8.0f, nullptr) == T12_OK && pack_on_gpu(stage, M, K, w);
-        (void)hipFree(stage);
-        if (!ok) engine_fail("synthetic tensor %s failed", n.c_str());
-    };
-    p.vector = [&](const std::string& n, float*& v, size_t k) {
-        float fill = n.find("norm") != std::string::npos ? 1.0f : 0.0f;
-        if (n.find("head_bias") != std::string::npos) fill = -3.0f;
-        if (n.find("w2t") != std::string::npos) fill = 0.01f;
-        if (n.find("w0") != std::string::npos) fill = -2.0f;
-        if (n.find("mlp.act") != std::string::npos) fill = 0.5f;
-        v = device_alloc<float>(k);
-        if (t12_fill_f32(v, k, fill, nullptr) != T12_OK) engine_fail("synthetic vector %s failed", n.c_str());
-    };
-    p.table = [&](const std::string& n, int16_t*& v, size_t k) {
-        v = device_alloc<int16_t>(k);
-        if (t12_synth_normal_bf16(v, k, ++s, 0.02f, 0.0f, 0.0f, nullptr) != T12_OK) engine_fail("synthetic table %s failed", n.c_str());
-    };
     try {
-        walk(c, m, data_of(m), p);
-        if (!gpu_ok(hipDeviceSynchronize(), "synthetic model")) engine_fail("synthetic model failed");
+        part_store::synthesize([&](const Parts& p) { walk(c, m, data_of(m), p); }, seed, p_outlier, [](const std::string& n) {
+            if (n.find("head_bias") != std::string::npos) return -3.0f;
+            if (n.find("w2t") != std::string::npos) return 0.01f;
+            if (n.find("w0") != std::string::npos) return -2.0f;
+            if (n.find("mlp.act") != std::string::npos) return 0.5f;
+            return n.find("norm") != std::string::npos ? 1.0f : 0.0f;
+        });
         derive(m);
     } catch (...) {
         release(m);

@@ -1,17 +1,12 @@
 // The layer stack of Gamilorn models (gamilorn.h): what a state holds, and a pass of rows through the layers.
 //
 // A state owns per layer a ring cache of keys and values and a pair of recurrent states for every sequence region
-// (t12_mixers.h).  A pass works on rows: one token of every sequence (decode), or consecutive tokens of one sequence
-// (prompt).  The recurrent states are read from one of the pair and written to the other, so the newest step can be
-// taken back by turning the pair around (the pipelined decode loop runs one step past an end-of-stream token).
+// (t12_mixers.h).  Regions, rows and the turning of the pair: regions.h.
 #include <algorithm>
 #include <cstdio>
-#include <cstdlib>
 
-#include "family.h"
 #include "gamilorn.h"
-#include "model_store.h"
-#include "t12_abi.h"
+#include "regions.h"
 #include "t12_glue.h"
 
 namespace gamilorn {
@@ -22,17 +17,9 @@ constexpr int kOverlapRows = 128;                // from this many prompt rows o
 constexpr float kUnitEps = 1e-6f;                // under the root of a key's length
 constexpr float kDecayRate = 0.60653065971263342f;   // exp(-1/2)
 
-struct State : StateCommon {
-    bool f32 = false;
-    bool per_seq = false;                        // false: all rows of the batch share region 0 (lock-step copies)
-    int rows = 0;                                // rows a pass can carry
-    int max_seq = 0;
+struct State : RegionState {
     std::vector<T12WindowAttn> attn;             // per layer, with the cache
     std::vector<T12DeltaRule> delta;             // per layer, with the states
-    std::vector<int> absorbed;                   // per region: tokens its recurrent states have seen
-    std::vector<int> parity;                     // per region: which of the pair is current
-    std::vector<void*> owned;                    // everything below and the caches
-    T12Row* d_rows = nullptr;
     float* in = nullptr;                         // [rows, in_rows]
     float* up = nullptr;                         // [rows, ff]
     float* work = nullptr;                       // delta rule
@@ -47,15 +34,13 @@ struct State : StateCommon {
 
 State* state_of(const InferenceState* s) { return (State*)(StateCommon*)s->impl; }
 
-// Every tensor can take the decode-GEMV with fused prologues and epilogues.
 bool fused_b1_eligible(const Model* model)
 {
     const Data& d = *data_of(model);
-    if (d.config.width % 16 || d.config.width > 8192 || !exp_ok(model->output_proj)) return false;
+    if (!region_norm_width(d.config.width) || !exp_ok(model->output_proj)) return false;
     for (const Layer& L : d.layers) {
-        const int oc = L.c.out_cols();
-        if (oc % 16 || oc > 81920 || !exp_ok(L.w_in) || !exp_ok(L.w_out)) return false;
-        if (L.c.ff && (L.c.ff % 16 || L.c.ff > 81920 || !exp_ok(L.up) || !exp_ok(L.down))) return false;
+        if (!region_fused_tensor(L.w_in) || !region_fused_tensor(L.w_out)) return false;
+        if (L.c.ff && (!region_fused_tensor(L.up) || !region_fused_tensor(L.down))) return false;
     }
     return true;
 }
@@ -69,11 +54,8 @@ InferenceState* create(Model* model, const StateOptions& o)
         return nullptr;
     }
     auto* st = new State();
-    st->f32 = o.precision == PRECISION_FP32;
-    st->per_seq = o.per_sequence;
-    st->max_seq = o.per_sequence && o.max_seq_len > 0 ? o.max_seq_len : model->max_seq_len;
-    st->rows = std::max(o.batch_size, std::min(o.prompt_rows > 0 ? o.prompt_rows : kPromptRows, st->max_seq));
-    const int regions = o.per_sequence ? o.batch_size : 1;
+    st->shape(o, model->max_seq_len, kPromptRows);
+    const int regions = st->regions();
     const size_t R = (size_t)st->rows, el = st->f32 ? 4 : 2;
 
     // sizes first: refuse what does not fit
@@ -128,17 +110,8 @@ InferenceState* create(Model* model, const StateOptions& o)
         return nullptr;
     }
     InferenceState* s = new_state(model, o.batch_size, st->rows, st);
-    auto own = [&](size_t bytes) {
-        void* p = nullptr;
-        check_gpu(hipMalloc(&p, std::max<size_t>(bytes, 16)), "hipMalloc");
-        st->owned.push_back(p);
-        return p;
-    };
-    auto zeroed = [&](size_t bytes) {
-        void* p = own(bytes);
-        check_gpu(hipMemsetAsync(p, 0, bytes, s->stream), "hipMemsetAsync");
-        return p;
-    };
+    auto own = [&](size_t bytes) { return st->own(bytes); };
+    auto zeroed = [&](size_t bytes) { return st->own_zeroed(bytes, s->stream); };
     for (size_t i = 0; i < d.layers.size(); i++) {
         st->attn[i].k = zeroed(regions * st->attn[i].k_elems * el);
         st->attn[i].v = zeroed(regions * st->attn[i].v_elems * el);
@@ -146,8 +119,6 @@ InferenceState* create(Model* model, const StateOptions& o)
     }
     check_gpu(hipEventCreateWithFlags(&st->fork, hipEventDisableTiming), "event");
     check_gpu(hipEventCreateWithFlags(&st->join, hipEventDisableTiming), "event");
-    st->absorbed.assign(regions, 0);
-    st->parity.assign(regions, 0);
     st->d_rows = (T12Row*)own(R * sizeof(T12Row));
     st->in = (float*)own(R * in * 4);
     st->up = (float*)own(R * ff * 4);
@@ -158,8 +129,7 @@ InferenceState* create(Model* model, const StateOptions& o)
     if (!st->f32) {
         st->step_ws = (float*)own(t12_parallel_step_ws_floats() * sizeof(float));
         st->step_count = (int*)zeroed(T12_STEP_MAX_ITEMS * sizeof(int));
-        const char* nofuse = getenv("TURBO_NO_FUSE");
-        st->fused_b1 = !(nofuse && nofuse[0] == '1') && o.batch_size == 1 && fused_b1_eligible(model);
+        st->fused_b1 = !region_no_fuse() && o.batch_size == 1 && fused_b1_eligible(model);
     }
     check_gpu(hipMalloc((void**)&s->hidden, R * c.width * 4), "hipMalloc");
     check_gpu(hipMalloc((void**)&s->hidden2, R * c.width * 4), "hipMalloc");
@@ -173,25 +143,6 @@ void release_state(InferenceState* s)
     for (void* p : st->owned) (void)hipFree(p);
     for (hipEvent_t e : {st->fork, st->join})
         if (e) (void)hipEventDestroy(e);
-}
-
-int max_positions(const InferenceState* s) { return state_of(s)->max_seq; }
-
-// A region's recurrent states only go forward: the next token must be the one after what they have absorbed, or the
-// first of a new sequence (which the kernels start from zero).
-void enter(State* st, int region, int position)
-{
-    if (position == 0) st->absorbed[region] = 0;
-    if (st->absorbed[region] != position)
-        engine_fail("position %d: the recurrent state of this sequence stands at %d (it continues there or restarts at 0)", position,
-                    st->absorbed[region]);
-}
-
-void linear(const CompressedWeight& w, float* out, int out_stride, const void* act, int K, int R, const State* st, hipStream_t q)
-{
-    T12Segment g = seg_of(w, out, out_stride);
-    if (st->f32) must(t12_gemm_f32(&g, 1, (const float*)act, K, out_stride, K, R, 0, q), "32-bit linear");
-    else run_linear(&g, 1, (const int16_t*)act, K, R, q);
 }
 
 // act = xIELU(up . h): in the GEMM's epilogue, in the sum over its K splits, or on its own.
@@ -210,7 +161,7 @@ void up_activation(State* st, const Layer& L, int n, int R, hipStream_t q)
             return;
         }
     } else {
-        linear(L.up, st->up, ff, st->h, n, R, st, q);
+        region_linear(L.up, st->up, ff, st->h, n, R, st->f32, q);
     }
     must(t12_act(st->up, &L.xielu, st->act, st->f32, (size_t)R * ff, q), "activation");
 }
@@ -221,8 +172,7 @@ void close_block(const CompressedWeight& w, const void* act, int K, const float*
 {
     const int n = w.M;
     if (st->f32) {
-        T12Segment g = seg_of(w, cur, n);
-        must(t12_gemm_f32(&g, 1, (const float*)act, K, n, K, R, 1, q), "32-bit linear");
+        region_linear_add_f32(w, cur, act, K, R, q);
         must(t12_rms_norm_f32(cur, norm, (float*)st->h, n, eps, R, q), "norm");
         return;
     }
@@ -238,7 +188,7 @@ void close_block(const CompressedWeight& w, const void* act, int K, const float*
 
 void head(InferenceState* s, State* st, const Config& c, const void* act, int R, float* out)
 {
-    linear(s->model->output_proj, out, c.vocab, act, c.width, R, st, s->stream);
+    region_linear(s->model->output_proj, out, c.vocab, act, c.width, R, st->f32, s->stream);
     const T12Act cap = {T12_ACT_SOFTCAP, c.softcap, 0.0f};
     if (c.softcap > 0.0f)
         must(t12_act(out, &cap, out, 1, (size_t)R * c.vocab, s->stream), "logit cap");
@@ -323,10 +273,13 @@ void pass_b1_fused(InferenceState* s, int position)
     else must(t12_gemv_norm(&g, 1, cur, nullptr, s->model->output_norm, c.eps, nullptr, n, q), "head decode-GEMV");
 }
 
-// R rows whose tokens are in s->d_tokens and whose row table is in st->d_rows; no row stands beyond max_position.
 void pass(InferenceState* s, int R, int run, int max_position, const LogitsRequest& lr)
 {
     State* st = state_of(s);
+    if (!run && st->fused_b1) {
+        pass_b1_fused(s, max_position);
+        return;
+    }
     const Data& d = *data_of(s->model);
     const Config& c = d.config;
     const int n = c.width;
@@ -340,7 +293,7 @@ void pass(InferenceState* s, int R, int run, int max_position, const LogitsReque
         const Layer& L = d.layers[i];
         const LayerConfig& k = L.c;
         const int ld = k.in_rows(), oc = k.out_cols();
-        linear(L.w_in, st->in, ld, st->h, n, R, st, q);
+        region_linear(L.w_in, st->in, ld, st->h, n, R, st->f32, q);
         mixers(s, L, i, R, run, max_position);
         const float* next = i + 1 < d.layers.size() ? d.layers[i + 1].norm1 : s->model->output_norm;
         close_block(L.w_out, st->cat, oc, k.ff ? L.norm2 : next, c.eps, R, st, cur, other, q);
@@ -360,76 +313,13 @@ void pass(InferenceState* s, int R, int run, int max_position, const LogitsReque
     }
 }
 
-void decode_step(InferenceState* s, const int* token_ids)
-{
-    State* st = state_of(s);
-    const int B = s->batch_size;
-    std::vector<T12Row> rows(B);
-    for (int b = 0; b < B; b++) {
-        const int region = st->per_seq ? b : 0;
-        if (!st->per_seq && s->positions[b] != s->positions[0])
-            engine_fail("the rows of a lock-step state must stand at one position");
-        enter(st, region, s->positions[b]);
-        rows[b] = {s->positions[b], region * 2 + st->parity[region]};
-    }
-    if (token_ids) check_gpu(hipMemcpyAsync(s->d_tokens, token_ids, B * sizeof(int), hipMemcpyHostToDevice, s->stream), "token copy");
-    must(t12_rows_list(st->d_rows, rows.data(), B, s->stream), "row table");
-    int max_position = 0;
-    for (const T12Row& r : rows) max_position = std::max(max_position, r.position);
-    LogitsRequest lr;
-    lr.mode = LOGITS_ALL;
-    if (st->fused_b1) pass_b1_fused(s, max_position);
-    else pass(s, B, 0, max_position, lr);
-    for (int& a : st->absorbed) a++;
-    for (int& p : st->parity) p ^= 1;
-    for (int b = 0; b < B; b++) s->positions[b]++;
-}
-
-void retract(InferenceState* s)
-{
-    State* st = state_of(s);
-    for (int& a : st->absorbed) a--;
-    for (int& p : st->parity) p ^= 1;
-    for (int b = 0; b < s->batch_size; b++) s->positions[b]--;
-}
-
-void prompt(InferenceState* s, const PromptPass& p)
-{
-    State* st = state_of(s);
-    const Config& c = data_of(s->model)->config;
-    const int region = st->per_seq ? p.seq : 0;
-    const size_t V = (size_t)c.vocab;
-    if (s->batch_size == 1 && p.n == 1) {                     // one token: the decode step
-        decode_step(s, p.tokens);
-        if (p.n_want > 0)
-            check_gpu(hipMemcpyAsync(p.logits, s->logits, V * sizeof(float), hipMemcpyDeviceToDevice, s->stream), "logits copy");
-        return;
-    }
-    const int rows = p.rows > 0 ? std::min(p.rows, st->rows) : st->rows;
-    float* last_row = s->logits + V * (st->per_seq ? p.seq : 0);
-    int taken = 0;
-    std::vector<int> picked;
-    for (int done = 0; done < p.n;) {
-        const int R = std::min(rows, p.n - done), pos = s->positions[p.seq];
-        enter(st, region, pos);
-        check_gpu(hipMemcpyAsync(s->d_tokens, p.tokens + done, R * sizeof(int), hipMemcpyHostToDevice, s->stream), "token copy");
-        must(t12_rows_run(st->d_rows, pos, region * 2 + st->parity[region], R, s->stream), "row table");
-        pass(s, R, 1, pos + R - 1, pass_logits(p, done, R, taken, c.vocab, last_row, picked));
-        st->absorbed[region] += R;
-        st->parity[region] ^= 1;
-        if (st->per_seq) s->positions[p.seq] += R;
-        else
-            for (int b = 0; b < s->batch_size; b++) s->positions[b] += R;
-        done += R;
-    }
-    for (int b = 1; !st->per_seq && p.n_want < 0 && b < s->batch_size; b++)
-        check_gpu(hipMemcpyAsync(s->logits + V * b, last_row, V * sizeof(float), hipMemcpyDeviceToDevice, s->stream), "logits copy");
-}
+void forward(InferenceState* s, const int* token_ids) { region_forward(s, token_ids, pass); }
+void prompt(InferenceState* s, const PromptPass& p) { region_prompt(s, p, pass); }
 
 }  // namespace
 }  // namespace gamilorn
 
 FamilyRun kGamilornRun = {
-    gamilorn::create, gamilorn::release_state, gamilorn::max_positions, gamilorn::decode_step, gamilorn::prompt, gamilorn::retract,
+    gamilorn::create, gamilorn::release_state, region_max_positions, gamilorn::forward, gamilorn::prompt, region_retract,
     nullptr,                                     // a recurrent state holds its whole past
 };

@@ -554,7 +554,7 @@ ModelFamily kLlamaFamily = {
 };
 
 namespace {
-const ModelFamily* const kFamilies[] = {&kGamilornFamily, &kLlamaFamily};
+const ModelFamily* const kFamilies[] = {&kGamilornFamily, &kDavasunFamily, &kLlamaFamily};
 }
 
 const ModelFamily& family_of(const Model* m) { return m->family ? *m->family : kLlamaFamily; }

@@ -88,6 +88,7 @@ struct GemmParams {
     uint16_t* out_bf16;                    // SwiGLU mode: bf16 [B, out_bf16_ld], silu(seg 2i) * seg 2i+1 of pair i
     int out_bf16_ld;
     float act_a, act_b;                    // EPI launches: the constants of the unary function
+    T12Glu glu = t12_silu_glu();           // SwiGLU mode: the unit
     int npair = 1;                         // SwiGLU mode: (gate, up) pairs of the launch; blk_start[i] = first tile of pair i
     // Rows per group known on the device only (the experts of a mixture-of-experts layer, counted by the routing
     // kernel): group_of_seg[s] picks an entry of dev_counts / dev_base, the segment's batch is dev_counts[.] and its
@@ -504,9 +505,8 @@ __device__ __forceinline__ bool gemm_mfma_body(const GemmParams& p, const int bt
 #pragma unroll
             for (int r = 0; r < 16; r++) {
                 const int b = b0 + (wb * FB + i) * 32 + 8 * (r >> 2) + 4 * lh + (r & 3);
-                const float g = acc[i][0][r];
                 if (m < M && b < B)
-                    ob[(size_t)b * p.out_bf16_ld + m] = t12_f32_to_bf16(g / (1.0f + expf(-g)) * acc[i][FM - 1][r]);
+                    ob[(size_t)b * p.out_bf16_ld + m] = t12_f32_to_bf16(t12_apply_glu(acc[i][0][r], acc[i][FM - 1][r], p.glu));
             }
         return true;
     }
@@ -868,7 +868,7 @@ __device__ __forceinline__ void gemm_dense16_body(const GemmParams& p, t12_f32x4
                 const int b = 16 * t + 4 * (l >> 4) + r, row = m0 + 16 * rg + (l & 15);
                 if (SWI) {
                     if (b < B && row < M)
-                        p.out_bf16[(size_t)b * p.out_bf16_ld + row] = t12_f32_to_bf16(v / (1.0f + expf(-v)) * u);
+                        p.out_bf16[(size_t)b * p.out_bf16_ld + row] = t12_f32_to_bf16(t12_apply_glu(v, u, p.glu));
                 } else if (b < B && row < M) outp[(size_t)b * sg.out_stride + row] = v;
             }
     }
@@ -1151,16 +1151,24 @@ int t12_gemm(const T12Segment* segs, int nseg, const void* act_bf16, int act_str
 int t12_gemm_swiglu(const T12Segment* gate, const T12Segment* up, const void* act_bf16, int act_stride, int K, int B,
                     void* out_bf16, int out_stride, void* stream)
 {
-    T12_REQUIRE(gate && up && act_bf16 && out_bf16, "t12_gemm_swiglu: null operand");
-    T12_REQUIRE(K >= 1 && B >= 1 && act_stride >= K, "t12_gemm_swiglu: K %d, B %d or act_stride %d invalid", K, B, act_stride);
-    T12_REQUIRE(gate->M >= 1 && gate->M == up->M, "t12_gemm_swiglu: gate has %d rows, up has %d", gate->M, up->M);
-    T12_REQUIRE(out_stride >= gate->M, "t12_gemm_swiglu: out_stride %d < M %d", out_stride, gate->M);
+    const T12Glu silu = t12_silu_glu();
+    return t12_gemm_glu(gate, up, &silu, act_bf16, act_stride, K, B, out_bf16, out_stride, stream);
+}
+
+// The same with any gated linear unit.
+int t12_gemm_glu(const T12Segment* gate, const T12Segment* up, const T12Glu* glu, const void* act_bf16, int act_stride, int K, int B,
+                 void* out_bf16, int out_stride, void* stream)
+{
+    T12_REQUIRE(gate && up && glu && act_bf16 && out_bf16, "t12_gemm_glu: null operand");
+    T12_REQUIRE(K >= 1 && B >= 1 && act_stride >= K, "t12_gemm_glu: K %d, B %d or act_stride %d invalid", K, B, act_stride);
+    T12_REQUIRE(gate->M >= 1 && gate->M == up->M, "t12_gemm_glu: gate has %d rows, up has %d", gate->M, up->M);
+    T12_REQUIRE(out_stride >= gate->M, "t12_gemm_glu: out_stride %d < M %d", out_stride, gate->M);
     const T12Segment* two[2] = {gate, up};
     bool fast = (K % KC == 0) && (act_stride % 8 == 0) && ((uintptr_t)act_bf16 % 16 == 0) && B > 64;
     for (const T12Segment* g : two) {
-        T12_REQUIRE(g->sm && g->gr, "t12_gemm_swiglu: a plane is null");
-        T12_REQUIRE(!g->row_off || (g->cols && g->correct && g->wrong), "t12_gemm_swiglu: row_off without lists");
-        T12_REQUIRE(g->base_exp >= -1 && g->base_exp <= 254, "t12_gemm_swiglu: base_exp %d out of range", g->base_exp);
+        T12_REQUIRE(g->sm && g->gr, "t12_gemm_glu: a plane is null");
+        T12_REQUIRE(!g->row_off || (g->cols && g->correct && g->wrong), "t12_gemm_glu: row_off without lists");
+        T12_REQUIRE(g->base_exp >= -1 && g->base_exp <= 254, "t12_gemm_glu: base_exp %d out of range", g->base_exp);
         if (g->base_exp < 0 || g->base_exp > 240) fast = false;
     }
     // 5 .. 8 batch rows: the whole-row sweep over 32 rows of gate and the same rows of up per workgroup.  Measured on
@@ -1173,6 +1181,7 @@ int t12_gemm_swiglu(const T12Segment* gate, const T12Segment* up, const void* ac
     if (sweep) {
         const int rg = 4;
         GemmParams p;
+        p.glu = *glu;
         p.seg[0] = *gate;
         p.seg[1] = *up;
         p.nseg = 2;
@@ -1191,13 +1200,14 @@ int t12_gemm_swiglu(const T12Segment* gate, const T12Segment* up, const void* ac
         p.out_bf16_ld = out_stride;
         hipStream_t st = (hipStream_t)stream;
         hipLaunchKernelGGL((gemm_dense16_swiglu_kernel<8, 2, 4>), dim3(sets), dim3(512), 0, st, p);
-        T12_CHECK_LAUNCH("t12_gemm_swiglu(dense16)");
+        T12_CHECK_LAUNCH("t12_gemm_glu(dense16)");
         return T12_OK;
     }
     const int tiles = (gate->M + TM / 2 - 1) / (TM / 2);
     const int btiles = B > 128 ? (B + 255) / 256 : 1;
     if (!fast || tiles * btiles * 4 < 256 * 3) return 1;      // would need a K split: partial sums cannot be gated
     GemmParams p;
+    p.glu = *glu;
     p.seg[0] = *gate;
     p.seg[1] = *up;
     p.nseg = 2;

@@ -1,4 +1,5 @@
-// Layer pieces around the mixers: embedding with learned positions, the 32-bit RMSNorm, unary activations.
+// Layer pieces around the mixers: embeddings (learned positions, normed), the 32-bit RMSNorm, norms around sublayers, unary
+// activations, gated linear units.
 
 #include "t12_act.h"
 #include "t12_device.h"
@@ -17,6 +18,145 @@ __global__ __launch_bounds__(256) void embed_positions_kernel(const uint16_t* __
     float v = t >= 0 && t < n_vocab ? t12_bf16_to_f32(table[(size_t)t * width + i]) : 0.0f;
     if (p >= 0 && p < n_positions) v += t12_bf16_to_f32(pos[(size_t)p * width + i]);
     out[(size_t)r * width + i] = v;
+}
+
+// Sum over a workgroup of whole waves, in every thread; red holds a float per wave.
+__device__ __forceinline__ float block_sum(float v, float* red)
+{
+    v = t12_wave_sum(v);
+    __syncthreads();                                       // red may still be read
+    if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = v;
+    __syncthreads();
+    float s = 0.0f;
+    for (int w = 0; w < (int)blockDim.x / 64; w++) s += red[w];
+    return s;
+}
+
+__global__ __launch_bounds__(256) void embed_norm_kernel(const uint16_t* __restrict__ table, int n_vocab, const int* __restrict__ tokens,
+                                                         const float* __restrict__ w, float eps, float* __restrict__ out, int width)
+{
+    __shared__ float red[4];
+    const int t = tokens[blockIdx.x];
+    const bool known = t >= 0 && t < n_vocab;
+    const uint16_t* row = table + (size_t)(known ? t : 0) * width;
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < width; i += 256) {
+        const float v = t12_bf16_to_f32(row[i]);
+        ss += v * v;
+    }
+    const float rn = known ? 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps) : 0.0f;
+    for (int i = threadIdx.x; i < width; i += 256) out[(size_t)blockIdx.x * width + i] = t12_bf16_to_f32(row[i]) * rn * w[i];
+}
+
+// One workgroup per row; a thread's values stay in registers between the two norms (width <= 8 x threads x ITEMS).  y
+// values: the sum of nsplit partial rows, or y itself.
+struct PostNormParams {
+    const float* y;
+    int nsplit;
+    size_t split_stride;
+    int ld;
+    const float* residual;
+    const float* post_w;
+    const float* norm_w;
+    float eps;
+    float* x_out;
+    void* h;
+    int width;
+};
+template <bool F32, bool VEC>
+__global__ __launch_bounds__(1024) void post_norm_add_kernel(const PostNormParams p)
+{
+    constexpr int E = VEC ? 4 : 1, ITEMS = VEC ? 2 : 8;
+    __shared__ float red[16];
+    const size_t r = blockIdx.x;
+    const int step = blockDim.x * E;
+    float v[ITEMS][E];
+    float ss = 0.0f;
+#pragma unroll
+    for (int q = 0; q < ITEMS; q++) {
+        const int i = threadIdx.x * E + q * step;
+#pragma unroll
+        for (int e = 0; e < E; e++) v[q][e] = 0.0f;
+        if (i < p.width) {
+            const float* src = p.y + r * p.ld + i;
+            for (int z = 0; z < p.nsplit; z++) {
+                if (VEC) {
+                    const t12_f32x4 a = *(const t12_f32x4*)(src + z * p.split_stride);
+#pragma unroll
+                    for (int e = 0; e < E; e++) v[q][e] += a[e];
+                } else v[q][0] += src[z * p.split_stride];
+            }
+#pragma unroll
+            for (int e = 0; e < E; e++) ss += v[q][e] * v[q][e];
+        }
+    }
+    const float pn = 1.0f / sqrtf(block_sum(ss, red) / (float)p.width + p.eps);
+    ss = 0.0f;
+#pragma unroll
+    for (int q = 0; q < ITEMS; q++) {
+        const int i = threadIdx.x * E + q * step;
+        if (i < p.width) {
+#pragma unroll
+            for (int e = 0; e < E; e++) {
+                v[q][e] = p.residual[r * p.width + i + e] + v[q][e] * pn * p.post_w[i + e];
+                ss += v[q][e] * v[q][e];
+                p.x_out[r * p.width + i + e] = v[q][e];
+            }
+        }
+    }
+    const float rn = 1.0f / sqrtf(block_sum(ss, red) / (float)p.width + p.eps);
+#pragma unroll
+    for (int q = 0; q < ITEMS; q++) {
+        const int i = threadIdx.x * E + q * step;
+        if (i < p.width) {
+#pragma unroll
+            for (int e = 0; e < E; e++) {
+                const float h = v[q][e] * rn * p.norm_w[i + e];
+                if (F32) ((float*)p.h)[r * p.width + i + e] = h;
+                else ((uint16_t*)p.h)[r * p.width + i + e] = t12_f32_to_bf16(h);
+            }
+        }
+    }
+}
+
+// Any width: x_out carries the values between the passes.
+template <bool F32>
+__global__ __launch_bounds__(1024) void post_norm_add_wide_kernel(const PostNormParams p)
+{
+    __shared__ float red[16];
+    const size_t r = blockIdx.x;
+    float* x = p.x_out + r * p.width;
+    float ss = 0.0f;
+    for (int i = threadIdx.x; i < p.width; i += blockDim.x) {
+        float v = 0.0f;
+        for (int z = 0; z < p.nsplit; z++) v += p.y[z * p.split_stride + r * p.ld + i];
+        x[i] = v;                                          // (y itself, or another buffer: each thread its own places)
+        ss += v * v;
+    }
+    const float pn = 1.0f / sqrtf(block_sum(ss, red) / (float)p.width + p.eps);
+    ss = 0.0f;
+    for (int i = threadIdx.x; i < p.width; i += blockDim.x) {
+        const float v = p.residual[r * p.width + i] + x[i] * pn * p.post_w[i];
+        x[i] = v;
+        ss += v * v;
+    }
+    const float rn = 1.0f / sqrtf(block_sum(ss, red) / (float)p.width + p.eps);
+    for (int i = threadIdx.x; i < p.width; i += blockDim.x) {
+        const float h = x[i] * rn * p.norm_w[i];
+        if (F32) ((float*)p.h)[r * p.width + i] = h;
+        else ((uint16_t*)p.h)[r * p.width + i] = t12_f32_to_bf16(h);
+    }
+}
+
+template <bool F32>
+__global__ __launch_bounds__(256) void glu_kernel(const float* __restrict__ gate, const float* __restrict__ up, const T12Glu glu, void* out,
+                                                  size_t n)
+{
+    const size_t i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= n) return;
+    const float v = t12_apply_glu(gate[i], up[i], glu);
+    if (F32) ((float*)out)[i] = v;
+    else ((uint16_t*)out)[i] = t12_f32_to_bf16(v);
 }
 
 __global__ __launch_bounds__(256) void rms_norm_f32_kernel(const float* __restrict__ x, const float* __restrict__ w,
@@ -98,6 +238,52 @@ int t12_embed_positions(const void* table_bf16, int n_vocab, const void* pos_bf1
     hipLaunchKernelGGL(embed_positions_kernel, dim3((width + 255) / 256, n), dim3(256), 0, (hipStream_t)stream,
                        (const uint16_t*)table_bf16, n_vocab, (const uint16_t*)pos_bf16, n_positions, tokens, rows, out, width);
     T12_CHECK_LAUNCH("t12_embed_positions");
+    return T12_OK;
+}
+
+int t12_embed_norm(const void* table_bf16, int n_vocab, const int* tokens, const float* weight, float eps, float* out, int width,
+                   int n, void* stream)
+{
+    T12_REQUIRE(table_bf16 && n_vocab >= 1 && tokens && weight && out && width >= 1 && n >= 1, "t12_embed_norm: bad operands");
+    hipLaunchKernelGGL(embed_norm_kernel, dim3(n), dim3(256), 0, (hipStream_t)stream, (const uint16_t*)table_bf16, n_vocab, tokens, weight,
+                       eps, out, width);
+    T12_CHECK_LAUNCH("t12_embed_norm");
+    return T12_OK;
+}
+
+int t12_post_norm_add(const float* y, const T12GemmPartials* part, const float* residual, const float* post_w, const float* norm_w,
+                      float eps, float* x_out, void* h, int h_f32, int width, int n, void* stream)
+{
+    T12_REQUIRE((part ? part->ws != nullptr && part->nsplit >= 1 && part->ld >= width : y != nullptr) && residual && post_w && norm_w &&
+                    x_out && x_out != residual && h && width >= 1 && n >= 1,
+                "t12_post_norm_add: bad operands");
+    PostNormParams p = {part ? part->ws : y, part ? part->nsplit : 1, part ? part->split_stride : 0, part ? part->ld : width, residual,
+                        post_w, norm_w, eps, x_out, h, width};
+    hipStream_t st = (hipStream_t)stream;
+    auto aligned = [](const void* q) { return (uintptr_t)q % 16 == 0; };
+    if (width % 4 == 0 && width <= 8192 && p.ld % 4 == 0 && p.split_stride % 4 == 0 && aligned(p.y) && aligned(x_out)) {
+        const int threads = width <= 4096 ? (width / 4 + 63) / 64 * 64 : 1024;
+        if (h_f32) hipLaunchKernelGGL((post_norm_add_kernel<true, true>), dim3(n), dim3(threads), 0, st, p);
+        else hipLaunchKernelGGL((post_norm_add_kernel<false, true>), dim3(n), dim3(threads), 0, st, p);
+    } else if (width <= 8192) {
+        const int threads = (((width + 7) / 8 + 63) / 64) * 64;
+        if (h_f32) hipLaunchKernelGGL((post_norm_add_kernel<true, false>), dim3(n), dim3(threads), 0, st, p);
+        else hipLaunchKernelGGL((post_norm_add_kernel<false, false>), dim3(n), dim3(threads), 0, st, p);
+    } else {
+        if (h_f32) hipLaunchKernelGGL(post_norm_add_wide_kernel<true>, dim3(n), dim3(1024), 0, st, p);
+        else hipLaunchKernelGGL(post_norm_add_wide_kernel<false>, dim3(n), dim3(1024), 0, st, p);
+    }
+    T12_CHECK_LAUNCH("t12_post_norm_add");
+    return T12_OK;
+}
+
+int t12_glu(const float* gate, const float* up, const T12Glu* glu, void* out, int out_f32, size_t n, void* stream)
+{
+    T12_REQUIRE(gate && up && glu && out && n >= 1, "t12_glu: bad operands");
+    const dim3 grid((unsigned)((n + 255) / 256));
+    if (out_f32) hipLaunchKernelGGL(glu_kernel<true>, grid, dim3(256), 0, (hipStream_t)stream, gate, up, *glu, out, n);
+    else hipLaunchKernelGGL(glu_kernel<false>, grid, dim3(256), 0, (hipStream_t)stream, gate, up, *glu, out, n);
+    T12_CHECK_LAUNCH("t12_glu");
     return T12_OK;
 }
 

@@ -12,3 +12,14 @@ __device__ __forceinline__ float t12_apply_act(float z, float a, float b)
 }
 
 __device__ __forceinline__ float t12_sigmoid(float x) { return 1.0f / (1.0f + expf(-x)); }
+
+// Gated linear unit of a (gate, up) pair of sums.
+__device__ __forceinline__ float t12_apply_glu(float g, float u, const T12Glu& p)
+{
+    g = g > p.limit ? p.limit : g;
+    u = u > p.limit ? p.limit : u < -p.limit ? -p.limit : u;
+    return g / (1.0f + expf(-p.slope * g)) * (u + p.offset);
+}
+
+// What SiLU(gate) * up is in these terms.
+inline T12Glu t12_silu_glu() { return {__builtin_inff(), 1.0f, 0.0f}; }
