@@ -15,7 +15,9 @@ struct LatentParams {
     const T12Row* rows;
     int n, run;
     void* q;                               // [row][head][row_p]: the query in the latent's coordinates, then its rotated part
-    void* mean;                            // [row][head][rank_p]: weighted mean of the latents
+    void* mean;                            // [row][head][rank_p]: weighted mean of the latents; or, with parts, their
+    float2* parts;                         // [row][head][splits]: (largest score, sum of weights) of every stretch of keys, whose
+    int splits;                            // weighted sums are then fp32 [row][head][splits][rank_p] in mean
 };
 
 template <typename T>
@@ -26,6 +28,12 @@ template <>
 __device__ __forceinline__ uint16_t to_cache<uint16_t>(float v) { return t12_f32_to_bf16(v); }
 __device__ __forceinline__ float from_cache(float v) { return v; }
 __device__ __forceinline__ float from_cache(uint16_t v) { return t12_bf16_to_f32(v); }
+
+__device__ __forceinline__ uint32_t pack_bf16(float lo, float hi)
+{
+    typedef __attribute__((ext_vector_type(2))) float f2;
+    return __builtin_bit_cast(uint32_t, __builtin_convertvector((f2){lo, hi}, t12_bf16x2));
+}
 
 // Where element e of a position's row lies within the row.
 __device__ __forceinline__ int place(const T12LatentAttn& a, int position, int e)

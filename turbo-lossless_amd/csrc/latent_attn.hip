@@ -4,8 +4,13 @@
 // inner products with the cached latent (and the shared rotated part), and the weighted mean of the latents is multiplied with
 // the value projection at the end.  So attention runs over one shared "head" of rank + rot_dim channels whose values are the
 // first rank of them, and a token's cache is that one row.
+//
+// A step is three launches: the key projection of the queries (beside it, in workgroups of their own, the cache store and the
+// rotations), attention, the value projection with the gate.  All three run on the matrix cores for the sizes that have
+// instances; 32-bit states and other sizes take the general forms.
 
 #include <algorithm>
+#include <mutex>
 
 #include "latent_attn.h"
 #include "t12_host.h"
@@ -14,14 +19,14 @@ using namespace latent_attn;
 
 namespace {
 
-// ---- what a row stores and asks with.  One workgroup per row: the normed latent and the rotated key part into the cache; the
+// ---- what a row stores and asks with, by one workgroup of 256 threads: the normed latent and the rotated key part into the cache; the
 // rotated parts of the queries, and zeros in the padding, into the query rows.
 template <typename T>
-__global__ __launch_bounds__(256) void latent_store_kernel(const LatentParams p)
+__device__ __forceinline__ void store_row(const LatentParams& p, int r)
 {
     __shared__ float red[4];
     const T12LatentAttn& a = p.a;
-    const int r = blockIdx.x, tid = threadIdx.x, half = a.rot_dim / 2;
+    const int tid = threadIdx.x, half = a.rot_dim / 2;
     const T12Row row = p.rows[r];
     const float* x = p.in + (size_t)r * p.ld;
     const float* c = x + a.c_off;
@@ -29,6 +34,7 @@ __global__ __launch_bounds__(256) void latent_store_kernel(const LatentParams p)
     float ss = 0.0f;
     for (int i = tid; i < a.rank; i += 256) ss += c[i] * c[i];
     ss = t12_wave_sum(ss);
+    __syncthreads();                                       // red may still be read for the row before
     if ((tid & 63) == 0) red[tid >> 6] = ss;
     __syncthreads();
     const float rn = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)a.rank + a.eps);
@@ -58,10 +64,14 @@ __global__ __launch_bounds__(256) void latent_store_kernel(const LatentParams p)
     }
 }
 
+template <typename T>
+__global__ __launch_bounds__(256) void latent_store_kernel(const LatentParams p)
+{
+    store_row<T>(p, blockIdx.x);
+}
+
 // ---- a product per head: y[r, h, m] = sum_k W[h M + m, k] x[r, h, k].  General form: any sizes, one wave per sixteen outputs
 // of a (row, head); sums in fp32.
-template <typename T>
-struct HeadIn;                             // how a head's vector is read
 struct FromProjection {                    // fp32 projections of the pass, rounded to what the state computes in
     const float* in;
     int ld, off, head_ld;
@@ -71,12 +81,67 @@ struct FromProjection {                    // fp32 projections of the pass, roun
         const float v = in[(size_t)r * ld + off + h * head_ld + k];
         return round ? t12_bf16_to_f32(t12_f32_to_bf16(v)) : v;
     }
+    // eight consecutive elements; left: how many there are
+    __device__ __forceinline__ void at8(int r, int h, int k, int left, float (&v)[8]) const
+    {
+        const float* x = in + (size_t)r * ld + off + h * head_ld + k;
+        if (left >= 8 && (uintptr_t)x % 16 == 0) {
+            const t12_f32x4 a = *(const t12_f32x4*)x, b = *(const t12_f32x4*)(x + 4);
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] = e < 4 ? a[e & 3] : b[e & 3];
+            return;
+        }
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] = e < left ? x[e] : 0.0f;
+    }
 };
 template <typename T>
 struct FromRows {                          // mean latents [row][head][rank_p]
     const T* x;
     int heads, head_ld;
     __device__ __forceinline__ float at(int r, int h, int k) const { return from_cache(x[((size_t)r * heads + h) * head_ld + k]); }
+    __device__ __forceinline__ void at8(int r, int h, int k, int left, float (&v)[8]) const
+    {
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] = e < left ? at(r, h, k + e) : 0.0f;
+    }
+};
+struct FromParts {                         // sums of stretches of keys, put together here
+    const float* sums;
+    const float2* parts;
+    int heads, head_ld, splits;
+    __device__ __forceinline__ float at(int r, int h, int k) const
+    {
+        const size_t unit = (size_t)r * heads + h;
+        float top = -1e30f, total = 0.0f, v = 0.0f;
+        for (int z = 0; z < splits; z++) top = fmaxf(top, parts[unit * splits + z].x);
+        for (int z = 0; z < splits; z++) {
+            const float w = exp2f(parts[unit * splits + z].x - top);
+            total += w * parts[unit * splits + z].y;
+            v += w * sums[(unit * splits + z) * head_ld + k];
+        }
+        return t12_bf16_to_f32(t12_f32_to_bf16(v / total));
+    }
+    __device__ __forceinline__ void at8(int r, int h, int k, int left, float (&v)[8]) const
+    {
+        const size_t unit = (size_t)r * heads + h;
+        const float2* q = parts + unit * splits;
+        const float* x = sums + unit * splits * head_ld + k;          // (rows are padded: eight elements are always there)
+        float top = q[0].x, total = 0.0f;
+        for (int z = 1; z < splits; z++) top = fmaxf(top, q[z].x);
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] = 0.0f;
+        for (int z = 0; z < splits; z++) {
+            const float w = exp2f(q[z].x - top);
+            const t12_f32x4 a = *(const t12_f32x4*)(x + (size_t)z * head_ld), b = *(const t12_f32x4*)(x + (size_t)z * head_ld + 4);
+            total += w * q[z].y;
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] += w * (e < 4 ? a[e & 3] : b[e & 3]);
+        }
+        const float inv = 1.0f / total;
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] = e < left ? v[e] * inv : 0.0f;
+    }
 };
 
 template <typename IN, typename OUT>
@@ -104,6 +169,14 @@ struct ToQuery {
     T* q;
     int heads, row_p;
     __device__ __forceinline__ void put(int r, int h, int m, float v) const { q[((size_t)r * heads + h) * row_p + m] = to_cache<T>(v); }
+    // four consecutive outputs (bf16), of which `left` exist
+    __device__ __forceinline__ void put4(int r, int h, int m, int left, t12_f32x4 v) const
+    {
+        T* o = q + ((size_t)r * heads + h) * row_p + m;
+        if (left >= 4) *(uint2*)o = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+        else
+            for (int e = 0; e < left; e++) o[e] = to_cache<T>(v[e]);
+    }
 };
 template <typename T>
 struct ToGated {                           // times the head's sigmoid gate
@@ -115,7 +188,108 @@ struct ToGated {                           // times the head's sigmoid gate
     {
         out[(size_t)r * out_ld + h * vdim + m] = to_cache<T>(v * t12_sigmoid(in[(size_t)r * ld + g_off + h]));
     }
+    __device__ __forceinline__ void put4(int r, int h, int m, int left, t12_f32x4 v) const
+    {
+        v *= t12_sigmoid(in[(size_t)r * ld + g_off + h]);
+        T* o = out + (size_t)r * out_ld + h * vdim + m;
+        if (left >= 4 && (uintptr_t)o % 8 == 0) *(uint2*)o = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+        else
+            for (int e = 0; e < min(left, 4); e++) o[e] = to_cache<T>(v[e]);
+    }
 };
+
+// ---- the product per head on the matrix cores: K a multiple of 32, base_exp in 0..240.  Workgroup = 64 outputs of a head for
+// 16 NT rows, a wave sixteen outputs; a lane takes 32 consecutive columns of one weight row per 128-column block (two sign/mantissa
+// pieces, one of nibbles), which feed four MFMAs with the activations in the same order.  The accumulators start from the
+// escapes' corrections.  STORE: workgroups with blockIdx.y == heads store the rows of their tile (latent attention's cache) instead.
+// Dynamic LDS: activations, 16-byte units of eight columns (paired like the decoded weights) [unit][16 NT rows].
+template <int NT, bool STORE, typename IN, typename OUT>
+__global__ __launch_bounds__(256) void heads_matrix_kernel(T12Segment w, int heads, int M, int K, IN in, OUT out, int n, const LatentParams lp)
+{
+    extern __shared__ uint4 lds[];
+    constexpr int ROWS = 16 * NT;
+    const int r0 = blockIdx.x * ROWS, h = blockIdx.y, tid = threadIdx.x;
+    if (STORE && h == heads) {
+        for (int r = r0 + blockIdx.z; r < min(r0 + ROWS, n); r += gridDim.z) store_row<uint16_t>(lp, r);
+        return;
+    }
+    const int lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l = lane & 15, g4 = lane >> 4;
+    const int m0 = blockIdx.z * 64 + wave * 16, blocks = (K + 127) / 128, units = blocks * 16;
+    const size_t row = (size_t)h * M + min(m0 + l, M - 1);
+    const uint8_t* sm = w.sm + row * K;
+    const uint8_t* gr = w.gr + row * K / 2;
+    const uint32_t be2 = t12_opaque(((uint32_t)w.base_exp << 7) | ((uint32_t)w.base_exp << 23));
+    uint4 s0, s1, gg;
+    auto request = [&](int b) {                            // (columns past K: the row's first ones again, times zero)
+        const int k = b * 128 + 32 * g4, at = k < K ? k : 0;
+        s0 = *(const uint4*)(sm + at);
+        s1 = *(const uint4*)(sm + at + 16);
+        gg = *(const uint4*)(gr + at / 2);
+    };
+    request(0);
+    for (int i = tid; i < units * ROWS; i += 256) {
+        const int u = i % units, r = i / units;
+        float v[8];
+        if (u * 8 < K) in.at8(min(r0 + r, n - 1), h, u * 8, K - u * 8, v);
+        else {
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] = 0.0f;
+        }
+        lds[u * ROWS + r] = make_uint4(pack_bf16(v[0], v[4]), pack_bf16(v[1], v[5]), pack_bf16(v[2], v[6]), pack_bf16(v[3], v[7]));
+    }
+    __syncthreads();
+    t12_f32x4 acc[NT];
+#pragma unroll
+    for (int t = 0; t < NT; t++) acc[t] = (t12_f32x4)(0.0f);
+    if (w.row_off) {
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const int m = min(m0 + 4 * g4 + i, M - 1);
+            const size_t at = (size_t)h * M + m;
+            for (int q = w.row_off[at]; q < w.row_off[at + 1]; q++) {
+                const float delta = t12_bf16_to_f32((uint16_t)w.correct[q]) - t12_bf16_to_f32((uint16_t)w.wrong[q]);
+                const int k = w.cols[q], e = k & 7;
+#pragma unroll
+                for (int t = 0; t < NT; t++)
+                    acc[t][i] += delta * t12_bf16_to_f32(((const uint16_t*)(lds + (k >> 3) * ROWS + t * 16 + l))[(e & 3) * 2 + (e >> 2)]);
+            }
+        }
+    }
+    for (int b = 0; b < blocks; b++) {
+        const uint4 c0 = s0, c1 = s1, cg = gg;
+        request(min(b + 1, blocks - 1));
+        uint32_t d[4][4];
+        t12_decode8(c0.x, c0.y, cg.x, be2, d[0]);
+        t12_decode8(c0.z, c0.w, cg.y, be2, d[1]);
+        t12_decode8(c1.x, c1.y, cg.z, be2, d[2]);
+        t12_decode8(c1.z, c1.w, cg.w, be2, d[3]);
+#pragma unroll
+        for (int e = 0; e < 4; e++) {
+            const t12_bf16x8 a = __builtin_bit_cast(t12_bf16x8, make_uint4(d[e][0], d[e][1], d[e][2], d[e][3]));
+#pragma unroll
+            for (int t = 0; t < NT; t++)
+                acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                    a, __builtin_bit_cast(t12_bf16x8, lds[(b * 16 + 4 * g4 + e) * ROWS + t * 16 + l]), acc[t], 0, 0, 0);
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < NT; t++) {
+        const int r = r0 + t * 16 + l, m = m0 + 4 * g4;
+        if (r < n && m < M) out.put4(r, h, m, M - m, acc[t]);
+    }
+}
+
+bool matrix_product(const T12Segment& w, int K) { return K % 32 == 0 && K <= 512 && w.base_exp >= 0 && w.base_exp <= 240 && (!w.row_off || w.wrong); }
+
+template <bool STORE, typename IN, typename OUT>
+void launch_heads(const T12Segment& w, int M, int K, const IN& in, const OUT& out, const LatentParams& p, hipStream_t st)
+{
+    const int heads = p.a.heads, nt = p.n > 16 && (!STORE || K <= 384) ? 4 : 1, units = (K + 127) / 128 * 16;
+    const dim3 grid((p.n + 16 * nt - 1) / (16 * nt), heads + (STORE ? 1 : 0), (M + 63) / 64);
+    const size_t lds = (size_t)units * 16 * nt * 16;
+    if (nt == 4) hipLaunchKernelGGL((heads_matrix_kernel<4, STORE, IN, OUT>), grid, dim3(256), lds, st, w, heads, M, K, in, out, p.n, p);
+    else hipLaunchKernelGGL((heads_matrix_kernel<1, STORE, IN, OUT>), grid, dim3(256), lds, st, w, heads, M, K, in, out, p.n, p);
+}
 
 // ---- attention, general form: one workgroup per (row, head), any sizes, fp32 arithmetic.  Dynamic LDS: the query [row_p].
 template <typename T>
@@ -164,6 +338,230 @@ __global__ __launch_bounds__(256) void latent_general_kernel(const LatentParams 
     }
 }
 
+// ---- attention on the matrix cores.  Everything transposed, so that no operand is moved between lanes:
+//
+//   S^T = K Q^T    keys = A rows from LDS, columns -- (row, head) pairs -- = B from registers; lane (n, g4) = (lane % 16,
+//                  lane / 16) receives keys 4 g4 .. 4 g4 + 3 of both 16-key halves of a block for column n;
+//   P              softmax in fp32 with a running maximum per column; the weights enter the product as two bf16 (16 bits);
+//   O^T += C^T P^T the lane's eight weights are its B operand as they are; A = the block's latents turned around by the LDS's
+//                  transposing reads, four keys of one channel per read.
+//
+// Workgroup = CT x 2 waves on 16 CT columns: wave w has columns 16 (w % CT) ..., and of every two blocks the one w / CT.  Blocks
+// come into LDS as they lie in the cache (their pieces are already spread over the banks), the next two while two are worked on.
+// run: columns run over all (row, head) pairs of the sequence; else blockIdx.z is the row.  blockIdx.y: stretch of keys.
+// Dynamic LDS: 2 x 2 blocks.
+typedef __attribute__((ext_vector_type(4))) short s16x4;
+typedef __attribute__((address_space(3))) uint8_t lds_byte;
+
+template <int RP, int CT>
+__global__ __launch_bounds__(CT * 128) void latent_matrix_kernel(const LatentParams p)
+{
+    constexpr int DT = RP + 2, ET = RP * 2, ROWB = DT * 64, BLKB = BLK * ROWB, NW = CT * 2;
+    extern __shared__ uint4 lds4[];
+    uint8_t* lds = (uint8_t*)lds4;
+    const T12LatentAttn& a = p.a;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), n = lane & 15, g4 = lane >> 4;
+    const int ct = wave % CT, ph = wave / CT;
+    const T12Row row = p.rows[p.run ? 0 : blockIdx.z];
+    const int ncol = p.run ? p.n * a.heads : a.heads, first = blockIdx.x * CT * 16, col = first + ct * 16 + n;
+    const size_t unit = (p.run ? 0 : (size_t)blockIdx.z * a.heads) + min(col, ncol - 1);
+    const int pos = row.position + (p.run ? min(col, ncol - 1) / a.heads : 0);
+    const int last = row.position + (p.run ? (min(first + CT * 16, ncol) - 1) / a.heads : 0);
+    const int blocks = last / BLK + 1, per = ((blocks + 1) / 2 + p.splits - 1) / p.splits * 2;
+    const int b0 = min((int)blockIdx.y * per, blocks), b1 = min(b0 + per, blocks);
+    const uint8_t* cache = (const uint8_t*)a.cache + (size_t)(row.slot >> 1) * a.cache_elems * 2;
+    // one block is BLKB / 1024 pieces of a wave's load; the waves share the pieces of both blocks
+    auto request = [&](int b, int buf) {
+#pragma unroll
+        for (int i = 0; i < 2 * BLKB / 1024 / NW; i++) {
+            const int piece = wave + i * NW, which = piece / (BLKB / 1024), at = piece % (BLKB / 1024) * 1024;
+            const uint8_t* src = cache + (size_t)min(b + which, blocks - 1) * BLKB + at + lane * 16;
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
+                                             (__attribute__((address_space(3))) void*)(lds + (buf * 2 + which) * BLKB + at), 16, 0, 0);
+        }
+    };
+    static_assert(2 * BLKB / 1024 % NW == 0, "the waves share the pieces evenly");
+    if (b0 < b1) request(b0, 0);
+    t12_bf16x8 Q[DT];
+    const uint16_t* q = (const uint16_t*)p.q + unit * a.row_p + 8 * g4;
+#pragma unroll
+    for (int s = 0; s < DT; s++) Q[s] = *(const t12_bf16x8*)(q + s * 32);
+    t12_f32x4 acc[ET];
+#pragma unroll
+    for (int e = 0; e < ET; e++) acc[e] = (t12_f32x4)(0.0f);
+    float top = -1e30f, sum = 0.0f;
+    const float scale = a.scale * 1.44269504088896341f;
+    // LDS offsets of this lane within a block: keys for the scores (two pieces, the rest by constants), turned reads (four)
+    int ko[2], vo[4];
+#pragma unroll
+    for (int s = 0; s < 2; s++) ko[s] = n * ROWB + ((4 * s + g4) ^ (n & 7)) * 16;
+    const int vk = 4 * g4 + (n >> 2);                      // key of this lane's turned reads
+#pragma unroll
+    for (int e = 0; e < 4; e++) vo[e] = vk * ROWB + ((2 * e + ((n & 3) >> 1)) ^ (vk & 7)) * 16 + (n & 1) * 8;
+    int buf = 0;
+    for (int b = b0; b < b1; b += 2) {
+        __builtin_amdgcn_s_waitcnt(0x0F70);                // vmcnt(0): the blocks have landed
+        __syncthreads();                                   // (the other buffer was last read before this barrier)
+        if (b + 2 < b1) request(b + 2, buf ^ 1);
+        const uint8_t* blk = lds + (buf * 2 + ph) * BLKB;
+        t12_f32x4 S[2];
+        S[0] = S[1] = (t12_f32x4)(0.0f);
+#pragma unroll
+        for (int s = 0; s < DT; s++)
+#pragma unroll
+            for (int u = 0; u < 2; u++)
+                S[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const t12_bf16x8*)(blk + ko[s & 1] + (s >> 1) * 128 + u * 16 * ROWB), Q[s],
+                                                               S[u], 0, 0, 0);
+        // keys past the column's position, and a whole block past the stretch, get no weight
+        const int left = b + ph < b1 ? pos - (b + ph) * BLK - 4 * g4 : -1;
+        float w[8], best = top;
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            w[i] = (i >> 2) * 16 + (i & 3) <= left ? S[i >> 2][i & 3] * scale : -INFINITY;
+            best = fmaxf(best, w[i]);
+        }
+        best = fmaxf(best, __shfl_xor(best, 16, 64));
+        best = fmaxf(best, __shfl_xor(best, 32, 64));
+        const float back = __builtin_amdgcn_exp2f(top - best);
+        const bool grew = __any(best > top);
+        top = best;
+        sum *= back;
+        uint32_t hi[4], lo[4];
+#pragma unroll
+        for (int i = 0; i < 8; i++) {
+            w[i] = __builtin_amdgcn_exp2f(w[i] - best);
+            sum += w[i];
+        }
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            hi[i] = pack_bf16(w[2 * i], w[2 * i + 1]);
+            lo[i] = pack_bf16(w[2 * i] - __builtin_bit_cast(float, hi[i] << 16), w[2 * i + 1] - __builtin_bit_cast(float, hi[i] & 0xFFFF0000u));
+        }
+        const t12_bf16x8 ph8 = __builtin_bit_cast(t12_bf16x8, make_uint4(hi[0], hi[1], hi[2], hi[3]));
+        const t12_bf16x8 pl8 = __builtin_bit_cast(t12_bf16x8, make_uint4(lo[0], lo[1], lo[2], lo[3]));
+        if (grew) {
+#pragma unroll
+            for (int e = 0; e < ET; e++) acc[e] *= back;
+        }
+#pragma unroll
+        for (int e = 0; e < ET; e++) {
+            struct { s16x4 h[2]; } v;
+#pragma unroll
+            for (int u = 0; u < 2; u++)
+                v.h[u] = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
+                    (__attribute__((address_space(3))) s16x4*)(lds_byte*)(blk + vo[e & 3] + (e >> 2) * 128 + u * 16 * ROWB));
+            const t12_bf16x8 vv = __builtin_bit_cast(t12_bf16x8, v);
+            acc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, ph8, acc[e], 0, 0, 0);
+            acc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pl8, acc[e], 0, 0, 0);
+        }
+        buf ^= 1;
+    }
+    // the two waves of a column tile, put together through LDS
+    sum += __shfl_xor(sum, 16, 64);
+    sum += __shfl_xor(sum, 32, 64);
+    __syncthreads();
+    float2* ml = (float2*)lds;                             // [NW][16]
+    if (g4 == 0) ml[wave * 16 + n] = make_float2(top, sum);
+    __syncthreads();
+    const float2 theirs = ml[(wave + CT) % NW * 16 + n];
+    const float both = fmaxf(top, theirs.x), mine = exp2f(top - both);
+    sum = sum * mine + theirs.y * exp2f(theirs.x - both);
+    const float inv = p.parts ? mine : mine / sum;
+    constexpr int EG = ET < 8 ? ET : 8;
+    t12_f32x4* red = (t12_f32x4*)(lds + 1024);             // [CT][EG][64]
+#pragma unroll
+    for (int e0 = 0; e0 < ET; e0 += EG) {
+        __syncthreads();
+        if (ph == 1) {
+#pragma unroll
+            for (int e = 0; e < EG; e++) red[(ct * EG + e) * 64 + lane] = acc[e0 + e] * inv;
+        }
+        __syncthreads();
+        if (ph == 0) {
+#pragma unroll
+            for (int e = 0; e < EG; e++) {
+                const t12_f32x4 s = acc[e0 + e] * inv + red[(ct * EG + e) * 64 + lane];
+                const int c = (e0 + e) * 16 + 4 * g4;
+                if (col >= ncol) continue;
+                if (p.parts) *(t12_f32x4*)((float*)p.mean + (unit * p.splits + blockIdx.y) * a.rank_p + c) = s;
+                else *(uint2*)((uint16_t*)p.mean + unit * a.rank_p + c) = make_uint2(pack_bf16(s[0], s[1]), pack_bf16(s[2], s[3]));
+            }
+        }
+    }
+    if (p.parts && ph == 0 && g4 == 0 && col < ncol) p.parts[unit * p.splits + blockIdx.y] = make_float2(both, sum);
+}
+
+constexpr int MAX_SPLITS = 32;
+constexpr int PART_UNITS = 16384;          // (row, head, stretch) sums a pass keeps when it keeps more than one stretch
+
+template <int RP, int CT>
+int launch_matrix(const LatentParams& p, int columns, hipStream_t st)
+{
+    constexpr size_t lds = (size_t)4 * BLK * (RP + 2) * 64;
+    if (lds > 64 * 1024) {
+        static std::once_flag once[16];                    // the attribute is per device
+        int dev = 0;
+        if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 16) dev = 0;
+        hipError_t e = hipSuccess;
+        std::call_once(once[dev], [&] { e = hipFuncSetAttribute((const void*)latent_matrix_kernel<RP, CT>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds); });
+        if (e != hipSuccess) {
+            t12_set_error("t12_latent_attention: cannot reserve %zu bytes of LDS", lds);
+            return T12_ELAUNCH;
+        }
+    }
+    hipLaunchKernelGGL((latent_matrix_kernel<RP, CT>), dim3((columns + CT * 16 - 1) / (CT * 16), p.splits, p.run ? 1 : p.n), dim3(CT * 128), lds, st, p);
+    return T12_OK;
+}
+
+template <int CT>
+int launch_matrix_rank(const LatentParams& p, int columns, hipStream_t st)
+{
+    switch (p.a.rank_p) {
+        case 64: return launch_matrix<2, CT>(p, columns, st);
+        case 128: return launch_matrix<4, CT>(p, columns, st);
+        case 256: return launch_matrix<8, CT>(p, columns, st);
+        default: return launch_matrix<16, CT>(p, columns, st);
+    }
+}
+
+int launch_fast(LatentParams p, int max_position, void* out, int out_ld, hipStream_t st)
+{
+    const T12LatentAttn& a = p.a;
+    const FromProjection q = {p.in, p.ld, a.q_off, a.dim + a.rot_dim, true};
+    const ToQuery<uint16_t> to = {(uint16_t*)p.q, a.heads, a.row_p};
+    if (matrix_product(*a.k_up, a.dim)) launch_heads<true>(*a.k_up, a.rank, a.dim, q, to, p, st);
+    else {
+        hipLaunchKernelGGL(latent_store_kernel<uint16_t>, dim3(p.n), dim3(256), 0, st, p);
+        hipLaunchKernelGGL((heads_general_kernel<FromProjection, ToQuery<uint16_t>>), dim3(p.n, a.heads, (a.rank + 63) / 64), dim3(256), 0, st,
+                           *a.k_up, a.heads, a.rank, a.dim, q, to, p.n);
+    }
+    // stretches of keys: as many as it takes to give every CU a workgroup, each at least four blocks
+    const int columns = p.run ? p.n * a.heads : a.heads, ct = columns > 32 ? 4 : columns > 16 ? 2 : 1;
+    const int groups = (columns + ct * 16 - 1) / (ct * 16) * (p.run ? 1 : p.n), blocks = max_position / BLK + 1;
+    p.splits = std::max(1, std::min({(256 + groups - 1) / groups, (blocks + 3) / 4, MAX_SPLITS, PART_UNITS / (p.n * a.heads)}));
+    const bool parts = !p.run || p.splits > 1;
+    if (!parts) p.parts = nullptr;
+    const int rc = ct == 4 ? launch_matrix_rank<4>(p, columns, st) : ct == 2 ? launch_matrix_rank<2>(p, columns, st) : launch_matrix_rank<1>(p, columns, st);
+    if (rc) return rc;
+    const ToGated<uint16_t> gated = {(uint16_t*)out, out_ld, a.vdim, p.in, p.ld, a.g_off};
+    const bool fast = matrix_product(*a.v_up, a.rank);
+    const dim3 general(p.n, a.heads, (a.vdim + 63) / 64);
+    if (parts) {
+        const FromParts mean = {(const float*)p.mean, p.parts, a.heads, a.rank_p, p.splits};
+        if (fast) launch_heads<false>(*a.v_up, a.vdim, a.rank, mean, gated, p, st);
+        else
+            hipLaunchKernelGGL((heads_general_kernel<FromParts, ToGated<uint16_t>>), general, dim3(256), 0, st, *a.v_up, a.heads, a.vdim, a.rank,
+                               mean, gated, p.n);
+    } else {
+        const FromRows<uint16_t> mean = {(const uint16_t*)p.mean, a.heads, a.rank_p};
+        if (fast) launch_heads<false>(*a.v_up, a.vdim, a.rank, mean, gated, p, st);
+        else
+            hipLaunchKernelGGL((heads_general_kernel<FromRows<uint16_t>, ToGated<uint16_t>>), general, dim3(256), 0, st, *a.v_up, a.heads, a.vdim,
+                               a.rank, mean, gated, p.n);
+    }
+    return T12_OK;
+}
+
 template <typename T>
 void launch_general(const LatentParams& p, void* out, int out_ld, hipStream_t st)
 {
@@ -190,13 +588,21 @@ int t12_latent_plan(T12LatentAttn* a, int max_positions, int rows)
                 "t12_latent_plan: impossible heads or sizes");
     T12_REQUIRE(max_positions >= 1 && rows >= 1 && (a->elem_bytes == 2 || a->elem_bytes == 4), "t12_latent_plan: %d positions, %d rows or element size %d invalid",
                 max_positions, rows, a->elem_bytes);
-    a->matrix = 0;
-    a->rank_p = (a->rank + 31) / 32 * 32;
-    a->row_p = a->rank_p + (a->rot_dim + 31) / 32 * 32;
+    a->matrix = a->elem_bytes == 2 && a->rank <= 512 && a->rot_dim <= 64;
+    if (a->matrix) {
+        a->rank_p = 64;
+        while (a->rank_p < a->rank) a->rank_p *= 2;
+        a->row_p = a->rank_p + 64;
+    } else {
+        a->rank_p = (a->rank + 31) / 32 * 32;
+        a->row_p = a->rank_p + (a->rot_dim + 31) / 32 * 32;
+    }
     const size_t blocks = (max_positions + BLK - 1) / BLK, el = a->elem_bytes;
     a->cache_elems = blocks * BLK * a->row_p;
-    const size_t q = (size_t)rows * a->heads * a->row_p * el, mean = (size_t)rows * a->heads * a->rank_p * el;
-    a->work_floats = (q + 15) / 16 * 4 + (mean + 15) / 16 * 4;
+    const size_t units = (size_t)rows * a->heads, q = units * a->row_p * el;
+    size_t mean = (units * a->rank_p * el + 3) / 4;
+    if (a->matrix) mean = std::max(units, (size_t)PART_UNITS) * (a->rank_p + 2);       // (fp32 sums of stretches, their weights)
+    a->work_floats = (q + 15) / 16 * 4 + (mean + 3) / 4 * 4;
     return T12_OK;
 }
 
@@ -223,6 +629,16 @@ int t12_latent_attention(const T12LatentAttn* a, const float* in, int ld, const 
     p.run = run;
     p.q = work;
     p.mean = work + ((size_t)n * a->heads * a->row_p * a->elem_bytes + 15) / 16 * 4;
+    if (a->matrix) {
+        T12_REQUIRE(a->elem_bytes == 2 && (a->rank_p == 64 || a->rank_p == 128 || a->rank_p == 256 || a->rank_p == 512) && a->row_p == a->rank_p + 64 &&
+                        (uintptr_t)a->cache % 16 == 0 && a->cache_elems % 8 == 0,
+                    "t12_latent_attention: t12_latent_plan has not been called, or the cache is not aligned");
+        p.parts = (float2*)((float*)p.mean + std::max((size_t)n * a->heads, (size_t)PART_UNITS) * a->rank_p);
+        const int rc = launch_fast(p, max_position, out, out_ld, st);
+        if (rc) return rc;
+        T12_CHECK_LAUNCH("t12_latent_attention");
+        return T12_OK;
+    }
     if (a->elem_bytes == 4) hipLaunchKernelGGL(latent_store_kernel<float>, dim3(n), dim3(256), 0, st, p);
     else hipLaunchKernelGGL(latent_store_kernel<uint16_t>, dim3(n), dim3(256), 0, st, p);
     if (a->elem_bytes == 4) launch_general<float>(p, out, out_ld, st);
