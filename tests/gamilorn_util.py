@@ -10,8 +10,8 @@ import numpy as np
 def bits_and_values(x):
     """bf16 bits of x and what they stand for, in float64."""
     synth = importlib.import_module("turbo_lossless_amd.synth")
-    b = synth.f32_to_bf16_bits(np.asarray(x, np.float32))
-    return b, synth.bf16_bits_to_f32(b).astype(np.float64)
+    b = synth.f32_to_bf16_bits(np.asarray(x, np.float32)).reshape(np.shape(x))
+    return b, synth.bf16_bits_to_f32(b).reshape(b.shape).astype(np.float64)
 
 
 def layer(heads=4, kv_heads=2, dim=32, vdim=32, window=20, keep=3, d_heads=2, d_dim=32, ff=96, scale=None, ls=0.9, rs=1.3):

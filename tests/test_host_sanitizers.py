@@ -1,5 +1,5 @@
 """CPU: the host-side parsers of the library (byte-level BPE tables, sentencepiece model reader, and the model
-directory checks load_model starts with: Llama directories, Gamilorn checkpoints with their JSON and safetensors readers) rebuilt with -fsanitize=address,undefined and run over well-formed,
+directory checks load_model starts with: Llama directories, Gamilorn and Davasun checkpoints with their JSON and safetensors readers) rebuilt with -fsanitize=address,undefined and run over well-formed,
 truncated and corrupted files.  A parser may refuse a file; it may not touch memory outside its buffers."""
 import importlib
 import io
@@ -143,12 +143,25 @@ def test_model_directory_check_under_sanitizers(t12, oracle, tmp_path, dir_exe):
     assert int(out.split()[1]) >= 1
 
 
-def test_checkpoint_check_under_sanitizers(t12, tmp_path, dir_exe):
-    from gamilorn_util import config, layer, tensors, write_checkpoint
+def small_gamilorn():
+    from gamilorn_util import config, layer, tensors
     cfg = config([layer(dim=16, vdim=16, d_heads=1, d_dim=8, ff=24), layer(heads=2, kv_heads=1, dim=8, vdim=24, d_dim=8, ff=0)], vocab=11,
                  width=24, positions=9)
+    return cfg, tensors(cfg, 3, 1), {"pos.bf16.bin": 9 * 24 * 2, "l0.mix.w2t.f32.bin": 3 * 2 * 8 * 4}
+
+
+def small_davasun():
+    from davasun_util import config, latent, mlstm, tensors
+    cfg = config([mlstm(heads=1, dim=8, vdim=8), latent(heads=1, dim=8, rot=4, vdim=8, rank=16, ff=24)], vocab=11, width=24, loop=(0, 1, 2))
+    return cfg, tensors(cfg, 1), {"embed.bf16.bin": 11 * 24 * 2, "embed.norm.f32.bin": 24 * 4}
+
+
+@pytest.mark.parametrize("make", [small_gamilorn, small_davasun])
+def test_checkpoint_check_under_sanitizers(t12, tmp_path, dir_exe, make):
+    from gamilorn_util import write_checkpoint
+    cfg, t, packed = make()
     good = tmp_path / "model"
-    write_checkpoint(str(good), cfg, tensors(cfg, 3, 1))
+    write_checkpoint(str(good), cfg, t)
     exe = dir_exe
     rng = random.Random(7)
     root = tmp_path / "mut"
@@ -169,8 +182,8 @@ def test_checkpoint_check_under_sanitizers(t12, tmp_path, dir_exe):
     bare = tmp_path / "bare"
     bare.mkdir()
     shutil.copy(good / "config.json", bare)
-    (bare / "pos.bf16.bin").write_bytes(b"\0" * (9 * 24 * 2))
-    (bare / "l0.mix.w2t.f32.bin").write_bytes(b"\0" * (3 * 2 * 8 * 4))
+    for name, size in packed.items():
+        (bare / name).write_bytes(b"\0" * size)
     dirs.append(str(bare))
     out = run(exe, ["dir", *dirs])
     assert int(out.split()[1]) >= 1

@@ -78,6 +78,28 @@ class DeltaRule(C.Structure):
                [("state_elems", C.c_size_t), ("work_elems", C.c_size_t), ("state", C.c_void_p)]
 
 
+class Glu(C.Structure):
+    """Mirror of T12Glu (include/t12_mixers.h)."""
+    _fields_ = [("limit", C.c_float), ("slope", C.c_float), ("offset", C.c_float)]
+
+
+class MatrixMemory(C.Structure):
+    """Mirror of T12MatrixMemory (include/t12_mixers.h)."""
+    _fields_ = [(n, C.c_int) for n in ("heads", "dim", "vdim")] + \
+               [(n, C.c_float) for n in ("q_scale", "gate_cap", "den_eps", "out_eps")] + [("norm_w", C.c_void_p)] + \
+               [(n, C.c_int) for n in ("q_off", "k_off", "v_off", "g_off", "i_off", "f_off", "dim_p")] + \
+               [("state_elems", C.c_size_t), ("work_floats", C.c_size_t), ("state", C.c_void_p)]
+
+
+class LatentAttn(C.Structure):
+    """Mirror of T12LatentAttn (include/t12_mixers.h)."""
+    _fields_ = [(n, C.c_int) for n in ("heads", "dim", "rot_dim", "vdim", "rank")] + \
+               [("scale", C.c_float), ("eps", C.c_float), ("elem_bytes", C.c_int)] + \
+               [("k_up", C.POINTER(Segment)), ("v_up", C.POINTER(Segment)), ("norm_w", C.c_void_p), ("freqs", C.c_void_p)] + \
+               [(n, C.c_int) for n in ("q_off", "c_off", "g_off", "rank_p", "row_p", "matrix")] + \
+               [("cache_elems", C.c_size_t), ("work_floats", C.c_size_t), ("cache", C.c_void_p)]
+
+
 ACT_XIELU, ACT_SOFTCAP = 1, 2
 STEP_MAX_ITEMS = 512
 
@@ -193,6 +215,16 @@ _SIGS = {
     "t12_embed_positions": (_i, [_vp, _i, _vp, _i, _vp, _vp, _vp, _i, _i, _vp]),
     "t12_rms_norm_f32": (_i, [_vp, _vp, _vp, _i, C.c_float, _i, _vp]),
     "t12_act": (_i, [_vp, C.POINTER(Act), _vp, _i, C.c_size_t, _vp]),
+    "t12_embed_norm": (_i, [_vp, _i, _vp, _vp, C.c_float, _vp, _i, _i, _vp]),
+    "t12_post_norm_add": (_i, [_vp, C.POINTER(GemmPartials), _vp, _vp, _vp, C.c_float, _vp, _vp, _i, _i, _i, _vp]),
+    "t12_glu": (_i, [_vp, _vp, C.POINTER(Glu), _vp, _i, C.c_size_t, _vp]),
+    "t12_gemm_glu": (_i, [C.POINTER(Segment), C.POINTER(Segment), C.POINTER(Glu), _vp, _i, _i, _i, _vp, _i, _vp]),
+    "t12_gemv_glu": (_i, [C.POINTER(Segment), C.POINTER(Segment), C.POINTER(Glu), _vp, _vp, _vp, _vp, _vp, C.c_float, _vp, _i, _vp, _vp]),
+    "t12_gemv_post_norm": (_i, [C.POINTER(Segment), _i, _vp, _vp, _vp, _vp, C.c_float, _vp, _i, _vp]),
+    "t12_memory_plan": (_i, [C.POINTER(MatrixMemory), _i]),
+    "t12_matrix_memory": (_i, [C.POINTER(MatrixMemory), _vp, _vp, _i, _vp, _i, _i, _i, _vp, _vp, _i, _i, _vp]),
+    "t12_latent_plan": (_i, [C.POINTER(LatentAttn), _i, _i]),
+    "t12_latent_attention": (_i, [C.POINTER(LatentAttn), _vp, _i, _vp, _i, _i, _i, _vp, _vp, _i, _i, _vp]),
     "t12_window_plan": (_i, [C.POINTER(WindowAttn), _i, _i]),
     "t12_window_store": (_i, [C.POINTER(WindowAttn), _vp, _vp, _i, _vp, _i, _i, _vp]),
     "t12_window_attention": (_i, [C.POINTER(WindowAttn), _vp, _vp, _i, _vp, _i, _i, C.c_float, _vp, _i, _i, _vp]),
