@@ -36,6 +36,10 @@ Workloads (synthetic, seeded, random-init weights of the Llama-3.1-8B shape:
                   (parameter counts within a few percent): prompt of 2048 tokens at B = 1, greedy decoding at B = 1 and B = 64
                   from 1024 positions of context; `roofline` prices the weight stream of the largest size's B = 1 step.
 
+  davasun         prompt and decode throughput of the Davasun family (mLSTM layers and latent attention layers, norms around
+                  every sublayer) at two layer sizes beside the Gamilorn family with as many mixers of either kind and feed-forwards
+                  of the same weights; the same measurements.
+
   tokenizer       host only: one step = encoding ~1 MB of text (150 000 words of a 4000-word list) with the engine's
                   byte-level BPE tokenizer over the ~20 000 merges that build those words; `cpu_baseline` is the reference's rule restated literally (one pass over the
                   text per merge) on a 4 KB sample of the same text.
@@ -646,90 +650,142 @@ def gamilorn_sizes():
             ("width_4096_window_4096", *size(4096, 32, 8, 32, 14336, 4096), 64)]
 
 
-def run_gamilorn(args, t12, torch, dev):
-    """Both families through the same engine calls: prefill / prefill_rows, the pipelined greedy decode loop."""
-    import ctypes as C
-    import numpy as np
-    prompt_len, context, n_batch = 2048, 1024, 64
-
-    def weights(cfg, llama):
-        L, n = cfg["layers"][0], llama["n_embd"]
+def gamilorn_weights(cfg, rank):
+    """(weights of all layers, of the head)"""
+    n, total = cfg["width"], 0
+    for L in cfg["layers"]:
         a, b, ff = L["mixer"]["left"], L["mixer"]["right"], L["mlp"]["ff"]
         d = b["heads"] * b["dim"]
-        g = n * (a["heads"] * a["dim"] + a["kv_heads"] * (a["dim"] + a["vdim"]) + 5 * d + 64) + n * (a["heads"] * a["vdim"] + d) + 2 * n * ff
-        kv = llama["n_head_kv"] * (n // llama["n_head"])
-        head = n * llama["n_vocab"]
-        return g * llama["n_layer"] + head, (2 * n * n + 2 * n * kv + 3 * n * llama["n_ff"]) * llama["n_layer"] + head
+        total += n * (a["heads"] * a["dim"] + a["kv_heads"] * (a["dim"] + a["vdim"]) + 5 * d + rank) + n * (a["heads"] * a["vdim"] + d) + 2 * n * ff
+    return total, n * cfg["vocab"]
 
-    def measure(make, n_weights, vocab):
-        rng = np.random.default_rng(3)
-        tok = [int(x) for x in rng.integers(0, vocab, prompt_len)]
-        out = {"weights": n_weights}
-        one = make(1, 0)
-        arr = (C.c_int * prompt_len)(*tok)
 
-        def enter(n):
-            one.set_positions([0])
-            t12.check(t12.lib.t12_engine_prefill_rows(one.state, arr, n, 512), "prefill_rows")
-            one.sync()
-        for _ in range(max(args.warmup, 1)):
-            enter(prompt_len)
-        t0 = time.perf_counter()
-        for _ in range(args.steps):
-            enter(prompt_len)
-        ms = (time.perf_counter() - t0) * 1e3 / args.steps
-        out["prompt_tok_s"] = prompt_len / ms * 1e3
-        out["prompt_TFLOPs_of_the_linears"] = 2.0 * (n_weights - vocab * width) * prompt_len / ms / 1e9
-        enter(context)
-        one.decode(8)
-        n_dec = 64
-        t0 = time.perf_counter()
-        one.decode(n_dec)
-        ms = (time.perf_counter() - t0) * 1e3 / n_dec
-        out["decode_b1_ms"], out["decode_b1_tok_s"], out["decode_b1_weight_GBps"] = ms, 1e3 / ms, 1.5 * n_weights / ms / 1e6
-        lib_free(one)
-        many = make(n_batch, 2048)
-        for b in range(n_batch):
-            many.prefill(b, tok[:context])
-        many.decode_all(4)
-        t0 = time.perf_counter()
-        many.decode_all(24)
-        ms = (time.perf_counter() - t0) * 1e3 / 24
-        out["decode_b%d_ms" % n_batch], out["decode_b%d_tok_s" % n_batch] = ms, n_batch * 1e3 / ms
-        lib_free(many)
-        return out
+def llama_weights(c):
+    n, kv = c["n_embd"], c["n_head_kv"] * (c["n_embd"] // c["n_head"])
+    return (2 * n * n + 2 * n * kv + 3 * n * c["n_ff"]) * c["n_layer"], n * c["n_vocab"]
 
-    def lib_free(e):
+
+FAMILY_PROMPT, FAMILY_CONTEXT, FAMILY_BATCH = 2048, 1024, 64
+
+
+def measure_family(args, t12, handle, weights, vocab):
+    """Prompt and decode throughput of one model through the engine calls every family shares: prefill / prefill_rows, the
+    pipelined greedy decode loop.  weights: (of all layers as run, of the head)."""
+    import ctypes as C
+    import numpy as np
+    rng = np.random.default_rng(3)
+    tok = [int(x) for x in rng.integers(0, vocab, FAMILY_PROMPT)]
+    n_weights = sum(weights)
+    out = {"weights": n_weights}
+    one = t12.Engine(handle, 1, 0)
+    arr = (C.c_int * FAMILY_PROMPT)(*tok)
+
+    def free(e):
         t12.lib.t12_engine_free_state(e.state)
         e.state = None
 
-    sizes = {}
-    for name, cfg, llama, rank in gamilorn_sizes():
-        width = llama["n_embd"]
-        n_g, n_l = weights(cfg, llama)
-        legs = {}
-        for family, n_weights in (("gamilorn", n_g), ("llama", n_l)):
-            if family == "gamilorn":
-                h = t12.lib.t12_engine_create_synthetic_gamilorn(json.dumps(cfg).encode(), rank, 4100, 3e-4)
-            else:
-                h = t12.lib.t12_engine_create_synthetic(llama["n_vocab"], width, llama["n_head"], llama["n_head_kv"], llama["n_layer"],
-                                                        llama["n_ff"], 8192, 500000.0, 1e-5, 4100, 8192, 3e-4)
-            legs[family] = measure(lambda batch, seq: t12.Engine(h, batch, seq), n_weights, llama["n_vocab"])
-            t12.lib.t12_engine_free_model(h)
-        sizes[name] = legs
-    g = sizes["width_4096"]["gamilorn"]
+    def enter(n):
+        one.set_positions([0])
+        t12.check(t12.lib.t12_engine_prefill_rows(one.state, arr, n, 512), "prefill_rows")
+        one.sync()
+    for _ in range(max(args.warmup, 1)):
+        enter(FAMILY_PROMPT)
+    t0 = time.perf_counter()
+    for _ in range(args.steps):
+        enter(FAMILY_PROMPT)
+    ms = (time.perf_counter() - t0) * 1e3 / args.steps
+    out["prompt_tok_s"] = FAMILY_PROMPT / ms * 1e3
+    out["prompt_TFLOPs_of_the_linears"] = 2.0 * weights[0] * FAMILY_PROMPT / ms / 1e9
+    enter(FAMILY_CONTEXT)
+    one.decode(8)
+    n_dec = 64
+    t0 = time.perf_counter()
+    one.decode(n_dec)
+    ms = (time.perf_counter() - t0) * 1e3 / n_dec
+    out["decode_b1_ms"], out["decode_b1_tok_s"], out["decode_b1_weight_GBps"] = ms, 1e3 / ms, 1.5 * n_weights / ms / 1e6
+    free(one)
+    many = t12.Engine(handle, FAMILY_BATCH, 2048)
+    for b in range(FAMILY_BATCH):
+        many.prefill(b, tok[:FAMILY_CONTEXT])
+    many.decode_all(4)
+    t0 = time.perf_counter()
+    many.decode_all(24)
+    ms = (time.perf_counter() - t0) * 1e3 / 24
+    out["decode_b%d_ms" % FAMILY_BATCH], out["decode_b%d_tok_s" % FAMILY_BATCH] = ms, FAMILY_BATCH * 1e3 / ms
+    free(many)
+    t12.lib.t12_engine_free_model(handle)
+    return out
+
+
+def family_line(args, name, what, sizes, head, beside):
+    """The JSON line of a family workload; head: the size whose B = 1 decode rate is the value."""
+    g = sizes[head][name]
     return {
-        "metric": "tok/s of greedy decoding at B=1, Gamilorn family, four layers of width 4096 (split-12 weights); prompt and "
-                  "B=64 throughput and the Llama family at equal size alongside",
+        "metric": "tok/s of greedy decoding at B=1, %s; prompt and B=64 throughput and %s at equal size alongside" % (what, beside),
         "value": g["decode_b1_tok_s"], "unit": "tok/s", "n_gpus": 1, "steps": args.steps, "warmup": args.warmup,
         "ms_per_step": g["decode_b1_ms"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None,
         "dtype": "bf16", "data": "synthetic",
-        "config": {"workload": "gamilorn: prompt of %d tokens, decode from %d positions at B=1 and B=%d, four layers, vocab 32000" %
-                               (prompt_len, context, n_batch)},
+        "config": {"workload": "%s: prompt of %d tokens, decode from %d positions at B=1 and B=%d, vocab 32000" %
+                               (name, FAMILY_PROMPT, FAMILY_CONTEXT, FAMILY_BATCH)},
         "sizes": sizes,
         "roofline": {"bound": "hbm", "achieved": g["decode_b1_weight_GBps"], "peak": HBM_PEAK_GBS, "unit": "GB/s",
                      "frac": g["decode_b1_weight_GBps"] / HBM_PEAK_GBS, "traffic": None, "kernel": "whole B=1 decode step, weight planes"},
     }
+
+
+def run_gamilorn(args, t12, torch, dev):
+    sizes = {}
+    for name, cfg, llama, rank in gamilorn_sizes():
+        g = t12.lib.t12_engine_create_synthetic_gamilorn(json.dumps(cfg).encode(), rank, 4100, 3e-4)
+        legs = {"gamilorn": measure_family(args, t12, g, gamilorn_weights(cfg, rank), cfg["vocab"])}
+        h = t12.lib.t12_engine_create_synthetic(llama["n_vocab"], llama["n_embd"], llama["n_head"], llama["n_head_kv"], llama["n_layer"],
+                                                llama["n_ff"], 8192, 500000.0, 1e-5, 4100, 8192, 3e-4)
+        legs["llama"] = measure_family(args, t12, h, llama_weights(llama), llama["n_vocab"])
+        sizes[name] = legs
+    return family_line(args, "gamilorn", "Gamilorn family, four layers of width 4096 (split-12 weights)", sizes, "width_4096", "the Llama family")
+
+
+def davasun_sizes():
+    """(name, Davasun config, Gamilorn config, its decay rank).  A Gamilorn layer is an attention, a recurrence and a
+    feed-forward; beside it stand an mLSTM layer and a latent attention layer with the feed-forward, three matrices of two
+    thirds the width."""
+    base = {name: (cfg, rank) for name, cfg, _, rank in gamilorn_sizes()}
+
+    def size(width, m_heads, m_dim, m_vdim, heads, rank, ff, pairs=4, loop=None):
+        mlstm = {"type": "mlstm", "mixer": {"heads": m_heads, "dim": m_dim, "vdim": m_vdim, "gate_cap": 15.0}, "mlp": None}
+        latent = {"type": "latent_attention", "mlp": {"kind": "dense", "ff": ff, "limit": 7.0},
+                  "mixer": {"heads": heads, "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": rank, "scale": 192 ** -0.5,
+                            "rot": {"dims": 64, "base": 10000.0}}}
+        return {"architecture": "Davasun", "layers": [mlstm, latent] * pairs, "vocab": 32000, "width": width, "norm": {"eps": 1e-5},
+                "logit_scale": 1.0, "loop": loop}
+    return [("width_2048", size(2048, 4, 256, 512, 16, 256, 5504), *base["width_2048"]),
+            ("width_4096", size(4096, 8, 256, 512, 32, 512, 9600), *base["width_4096"])]
+
+
+def davasun_weights(cfg):
+    n, total = cfg["width"], 0
+    for L in cfg["layers"]:
+        c = L["mixer"]
+        hv = c["heads"] * c["vdim"]
+        if L["type"] == "mlstm":
+            total += n * (2 * c["heads"] * c["dim"] + 3 * hv + 2 * c["heads"])
+        else:
+            total += n * (c["heads"] * (c["dim"] + c["rot_dim"]) + c["kv_rank"] + c["rot_dim"] + c["heads"] + hv)
+            total += c["heads"] * c["kv_rank"] * (c["dim"] + c["vdim"])
+        total += 3 * n * L["mlp"]["ff"] if L["mlp"] else 0
+    return total, n * cfg["vocab"]
+
+
+def run_davasun(args, t12, torch, dev):
+    sizes = {}
+    for name, cfg, other, rank in davasun_sizes():
+        h = t12.lib.t12_engine_create_synthetic_davasun(json.dumps(cfg).encode(), 4100, 3e-4)
+        legs = {"davasun": measure_family(args, t12, h, davasun_weights(cfg), cfg["vocab"])}
+        g = t12.lib.t12_engine_create_synthetic_gamilorn(json.dumps(other).encode(), rank, 4100, 3e-4)
+        legs["gamilorn"] = measure_family(args, t12, g, gamilorn_weights(other, rank), other["vocab"])
+        sizes[name] = legs
+    return family_line(args, "davasun", "Davasun family, four mLSTM and four latent attention layers of width 4096 (split-12 weights)", sizes,
+                       "width_4096", "the Gamilorn family")
 
 
 def gemm_layer_leg(t12, torch, dev, cfg, weight_of, n_rot, cur, g, batches=(2, 4, 8, 16, 32, 64, 128, 256), iters=50,
@@ -1029,7 +1085,7 @@ def main():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=20)
     ap.add_argument("--warmup", type=int, default=3)
-    ap.add_argument("--workload", default="decode", choices=["decode", "gemv_stack_b1", "moe", "gemm_layers", "attention", "codec", "convert", "tokenizer", "gamilorn"])
+    ap.add_argument("--workload", default="decode", choices=["decode", "gemv_stack_b1", "moe", "gemm_layers", "attention", "codec", "convert", "tokenizer", "gamilorn", "davasun"])
     ap.add_argument("--prompt", type=int, default=128)
     ap.add_argument("--no-batch256", dest="batch256", action="store_false")
     ap.add_argument("--layers", type=int, default=LLAMA8B["n_layer"], help="debug: fewer layers (invalid as a result)")
@@ -1072,8 +1128,8 @@ def main():
     if args.workload == "codec":
         emit(run_codec(args, t12, torch, dev), json_fd)
         return
-    if args.workload == "gamilorn":
-        emit(run_gamilorn(args, t12, torch, dev), json_fd)
+    if args.workload in ("gamilorn", "davasun"):
+        emit((run_gamilorn if args.workload == "gamilorn" else run_davasun)(args, t12, torch, dev), json_fd)
         return
     if args.workload == "convert":
         emit(run_convert(args, t12, torch, dev), json_fd)

@@ -83,18 +83,11 @@ typedef struct T12Glu {
 } T12Glu;
 /* out[i] = glu(gate[i], up[i]), i < n; out_f32: fp32, else bf16. */
 int t12_glu(const float* gate, const float* up, const T12Glu* glu, void* out, int out_f32, size_t n, void* stream);
-/* t12_gemm_swiglu (t12_abi.h) and the t12_gemv_swiglu pair with any unit.  t12_gemv_glu takes bf16 activations, or (act_bf16
- * NULL) builds them in its prologue: x normed; with residual, x + residual normed; with post_w too, residual +
- * rmsnorm(x) * post_w normed.  hidden_out (may be NULL) receives the sum. */
+/* t12_gemm_swiglu and t12_gemv_swiglu (t12_abi.h) with any unit. */
 int t12_gemm_glu(const struct T12Segment* gate, const struct T12Segment* up, const T12Glu* glu, const void* act_bf16, int act_stride,
                  int K, int B, void* out_bf16, int out_stride, void* stream);
-int t12_gemv_glu(const struct T12Segment* gate, const struct T12Segment* up, const T12Glu* glu, const void* act_bf16, const float* x,
-                 const float* residual, const float* post_w, const float* norm_w, float eps, float* hidden_out, int K, void* out_bf16,
-                 void* stream);
-/* t12_gemv_norm (t12_abi.h) whose addend goes through a norm of its own: activations = bf16(rmsnorm(s) * norm_w),
- * s = residual + rmsnorm(x) * post_w (-> hidden_out when given; it may not alias x or residual). */
-int t12_gemv_post_norm(const struct T12Segment* segs, int nseg, const float* x, const float* residual, const float* post_w,
-                       const float* norm_w, float eps, float* hidden_out, int K, void* stream);
+int t12_gemv_glu(const struct T12Segment* gate, const struct T12Segment* up, const T12Glu* glu, const void* act_bf16, int K,
+                 void* out_bf16, void* stream);
 
 /* ---- windowed attention with sigmoid weights -------------------------------------------------------------------
  * Query head h reads key/value head h / (heads / kv_heads).  The query at position i sees the key at j <= i when
@@ -186,7 +179,7 @@ int t12_matrix_memory(const T12MatrixMemory* m, const float* in, const float* bi
  *
  * The cache of a region: blocks of 32 positions, position p in row p % 32; a row holds c [rank] padded (zeros) to rank_p, then
  * the rotated part padded to row_p - rank_p.  bf16 caches of sizes that have a matrix-core instance (rank_p 64, 128, 256
- * or 512, row_p = rank_p + 64) keep the row's 16-byte pieces in the order piece ^ (p % 8). */
+ * or 512, row_p = rank_p + 64) keep the row's 16-byte pieces in an order that spreads equal pieces of neighbouring positions over the banks. */
 typedef struct T12LatentAttn {
     int   heads, dim, rot_dim, vdim, rank;
     float scale, eps;

@@ -219,8 +219,7 @@ _SIGS = {
     "t12_post_norm_add": (_i, [_vp, C.POINTER(GemmPartials), _vp, _vp, _vp, C.c_float, _vp, _vp, _i, _i, _i, _vp]),
     "t12_glu": (_i, [_vp, _vp, C.POINTER(Glu), _vp, _i, C.c_size_t, _vp]),
     "t12_gemm_glu": (_i, [C.POINTER(Segment), C.POINTER(Segment), C.POINTER(Glu), _vp, _i, _i, _i, _vp, _i, _vp]),
-    "t12_gemv_glu": (_i, [C.POINTER(Segment), C.POINTER(Segment), C.POINTER(Glu), _vp, _vp, _vp, _vp, _vp, C.c_float, _vp, _i, _vp, _vp]),
-    "t12_gemv_post_norm": (_i, [C.POINTER(Segment), _i, _vp, _vp, _vp, _vp, C.c_float, _vp, _i, _vp]),
+    "t12_gemv_glu": (_i, [C.POINTER(Segment), C.POINTER(Segment), C.POINTER(Glu), _vp, _i, _vp, _vp]),
     "t12_memory_plan": (_i, [C.POINTER(MatrixMemory), _i]),
     "t12_matrix_memory": (_i, [C.POINTER(MatrixMemory), _vp, _vp, _i, _vp, _i, _i, _i, _vp, _vp, _i, _i, _vp]),
     "t12_latent_plan": (_i, [C.POINTER(LatentAttn), _i, _i]),

@@ -43,7 +43,6 @@ struct GemvParams {
     int act_stride;                        // bf16 elements between activation rows
     int out_ld;                            // elements between output rows (fp32 outputs and out_bf16)
     float act_a, act_b;                    // EPI launches: the constants of the unary function
-    const float* npost;                    // NORM 3: weight of the norm that nx goes through before it is added
     T12Glu glu = t12_silu_glu();           // SwiGLU mode: the unit
 };
 
@@ -112,7 +111,6 @@ __device__ __forceinline__ float lds_act_at(const uint4* lds_act, int k)
 // workgroup rebuilds them from the fp32 residual stream while its first weight tiles are in
 // flight -- the reference's (add_)rms_norm_bf16_batch kernels (engine/kernels.hip:355-442) as a
 // prologue.  K <= 16 * NW * 64.  Workgroup 0 also stores nx + nres for the residual path.
-// NORM 3: the addend is itself RMS-normed first, nres + rmsnorm(nx) * npost (decoders with a norm behind every sublayer).
 // EPI (T12_ACT_*): the unary function applied to every sum of a single-segment launch -- xIELU stored as bf16 to
 // p.out_bf16[m] (the front half of a feed-forward without a gate), the soft cap in place of the plain fp32 store.
 // MOE: one activation row per blockIdx.y, multiplied with the tensors of the expert slot_expert[blockIdx.y] names --
@@ -164,7 +162,7 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
     }
 
     // NORM: the same for the fp32 residual stream, its addend and the norm weights (8 columns per piece, 2 pieces per thread)
-    float4 npre[NORM ? 2 : 1][2], rpre[NORM >= 2 ? 2 : 1][2], wpre[NORM ? 2 : 1][2], ppre[NORM == 3 ? 2 : 1][2];
+    float4 npre[NORM ? 2 : 1][2], rpre[NORM == 2 ? 2 : 1][2], wpre[NORM ? 2 : 1][2];
     if (NORM != 0) {
 #pragma unroll
         for (int gi = 0; gi < 2; gi++) {
@@ -172,13 +170,9 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
             if (gi == 0 || NW * 64 * 8 < K) {                        // workgroup-uniform
                 npre[gi][0] = *(const float4*)(p.nx + k);
                 npre[gi][1] = *(const float4*)(p.nx + k + 4);
-                if (NORM >= 2) {
+                if (NORM == 2) {
                     rpre[gi][0] = *(const float4*)(p.nres + k);
                     rpre[gi][1] = *(const float4*)(p.nres + k + 4);
-                }
-                if (NORM == 3) {
-                    ppre[gi][0] = *(const float4*)(p.npost + k);
-                    ppre[gi][1] = *(const float4*)(p.npost + k + 4);
                 }
                 wpre[gi][0] = *(const float4*)(p.nw + k);
                 wpre[gi][1] = *(const float4*)(p.nw + k + 4);
@@ -242,25 +236,9 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
             lds_act[(q >> 7) * 128 + (q & 1) * 64 + ((q & 127) >> 1)] = t12_pair_acts(v);
         }
     } else {
-        __shared__ float red[NW], red0[NW];
+        __shared__ float red[NW];
         float v[2][8];
-        float ss = 0.0f, post = 1.0f;
-        if (NORM == 3) {                                   // the addend's own norm
-            float s0 = 0.0f;
-#pragma unroll
-            for (int gi = 0; gi < 2; gi++)
-                if ((tid + gi * NW * 64) * 8 < K) {
-                    const float4 a = npre[gi][0], b = npre[gi][1];
-                    s0 += a.x * a.x + a.y * a.y + a.z * a.z + a.w * a.w + b.x * b.x + b.y * b.y + b.z * b.z + b.w * b.w;
-                }
-            s0 = t12_wave_sum(s0);
-            if (lane == 0) red0[wave] = s0;
-            __syncthreads();
-            float t0 = 0.0f;
-#pragma unroll
-            for (int w = 0; w < NW; w++) t0 += red0[w];
-            post = 1.0f / sqrtf(t0 / (float)K + p.eps);
-        }
+        float ss = 0.0f;
 #pragma unroll
         for (int gi = 0; gi < 2; gi++) {
             const int k = (tid + gi * NW * 64) * 8;
@@ -270,12 +248,7 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
                 const float4 a = npre[gi][0], b = npre[gi][1];
                 v[gi][0] = a.x; v[gi][1] = a.y; v[gi][2] = a.z; v[gi][3] = a.w;
                 v[gi][4] = b.x; v[gi][5] = b.y; v[gi][6] = b.z; v[gi][7] = b.w;
-                if (NORM == 3) {
-                    const float4 c = ppre[gi][0], d = ppre[gi][1];
-                    v[gi][0] *= post * c.x; v[gi][1] *= post * c.y; v[gi][2] *= post * c.z; v[gi][3] *= post * c.w;
-                    v[gi][4] *= post * d.x; v[gi][5] *= post * d.y; v[gi][6] *= post * d.z; v[gi][7] *= post * d.w;
-                }
-                if (NORM >= 2) {
+                if (NORM == 2) {
                     const float4 c = rpre[gi][0], d = rpre[gi][1];
                     v[gi][0] += c.x; v[gi][1] += c.y; v[gi][2] += c.z; v[gi][3] += c.w;
                     v[gi][4] += d.x; v[gi][5] += d.y; v[gi][6] += d.z; v[gi][7] += d.w;
@@ -618,15 +591,24 @@ extern "C" {
 int t12_gemv_swiglu(const T12Segment* gate, const T12Segment* up, const void* act_bf16, int K, void* out_bf16,
                     void* stream)
 {
-    T12_REQUIRE(gate && up && out_bf16, "t12_gemv_swiglu: null operand");
+    const T12Glu silu = t12_silu_glu();
+    return t12_gemv_glu(gate, up, &silu, act_bf16, K, out_bf16, stream);
+}
+
+// The same with any gated linear unit.
+int t12_gemv_glu(const T12Segment* gate, const T12Segment* up, const T12Glu* glu, const void* act_bf16, int K, void* out_bf16,
+                 void* stream)
+{
+    T12_REQUIRE(gate && up && glu && out_bf16, "t12_gemv_glu: null operand");
     T12Segment two[2] = {*gate, *up};
     int rc = validate(two, 2, act_bf16, K, false);
     if (rc) return rc;
-    T12_REQUIRE(gate->M == up->M, "t12_gemv_swiglu: gate has %d rows, up has %d", gate->M, up->M);
-    T12_REQUIRE(K % 16 == 0 && (K + 1023) / 1024 * 2048 <= 160 * 1024, "t12_gemv_swiglu: K %d must be a multiple of 16", K);
+    T12_REQUIRE(gate->M == up->M, "t12_gemv_glu: gate has %d rows, up has %d", gate->M, up->M);
+    T12_REQUIRE(K % 16 == 0 && (K + 1023) / 1024 * 2048 <= 160 * 1024, "t12_gemv_glu: K %d must be a multiple of 16", K);
     T12_REQUIRE(gate->base_exp >= 0 && gate->base_exp <= 240 && up->base_exp >= 0 && up->base_exp <= 240,
-                "t12_gemv_swiglu: base_exp outside 0..240 (use t12_gemv + launch_silu_mul_bf16_batch)");
+                "t12_gemv_glu: base_exp outside 0..240 (use t12_gemv and the unit on its own)");
     GemvParams p;
+    p.glu = *glu;
     p.seg[0] = two[0];
     p.seg[1] = two[1];
     p.nseg = 2;
@@ -720,68 +702,6 @@ int t12_gemv_act(const T12Segment* seg, const void* act_bf16, const float* x, co
     hipStream_t st = (hipStream_t)stream;
     if (act_bf16) return act->kind == T12_ACT_XIELU ? launch_act<0, T12_ACT_XIELU>(p, st) : launch_act<0, T12_ACT_SOFTCAP>(p, st);
     return act->kind == T12_ACT_XIELU ? launch_act<1, T12_ACT_XIELU>(p, st) : launch_act<1, T12_ACT_SOFTCAP>(p, st);
-}
-
-// y_s = W_s . bf16(rmsnorm(sum) * norm_w), sum = residual + rmsnorm(x) * post_w, both norms in the kernel's prologue.
-int t12_gemv_post_norm(const T12Segment* segs, int nseg, const float* x, const float* residual, const float* post_w, const float* norm_w,
-                       float eps, float* hidden_out, int K, void* stream)
-{
-    T12_REQUIRE(residual && post_w, "t12_gemv_post_norm: residual / post-norm weight is null");
-    int rc = validate(segs, nseg, x, K, true);
-    if (rc) return rc;
-    rc = check_norm_operands("t12_gemv_post_norm", segs, nseg, x, residual, norm_w, hidden_out, K);
-    if (rc) return rc;
-    GemvParams p;
-    for (int i = 0; i < nseg; i++) p.seg[i] = segs[i];
-    p.nseg = nseg;
-    p.K = K;
-    p.act = nullptr;
-    p.out_bf16 = nullptr;
-    p.add = nullptr;
-    p.nx = x;
-    p.nres = residual;
-    p.npost = post_w;
-    p.nw = norm_w;
-    p.hidden_out = hidden_out;
-    p.eps = eps;
-    return launch_plain_norm<3>(p, segs, nseg, (hipStream_t)stream);
-}
-
-int t12_gemv_glu(const T12Segment* gate, const T12Segment* up, const T12Glu* glu, const void* act_bf16, const float* x, const float* residual,
-                 const float* post_w, const float* norm_w, float eps, float* hidden_out, int K, void* out_bf16, void* stream)
-{
-    T12_REQUIRE(gate && up && glu && out_bf16, "t12_gemv_glu: null operand");
-    T12Segment two[2] = {*gate, *up};
-    int rc = validate(two, 2, act_bf16 ? act_bf16 : x, K, false);
-    if (rc) return rc;
-    T12_REQUIRE(gate->M == up->M, "t12_gemv_glu: gate has %d rows, up has %d", gate->M, up->M);
-    if (act_bf16) {
-        T12_REQUIRE(K % 16 == 0 && (K + 1023) / 1024 * 2048 <= 160 * 1024 && gate->base_exp >= 0 && gate->base_exp <= 240 &&
-                        up->base_exp >= 0 && up->base_exp <= 240,
-                    "t12_gemv_glu: K %d must be a multiple of 16 and base_exp within 0..240", K);
-    } else {
-        rc = check_norm_operands("t12_gemv_glu", two, 2, x, residual, norm_w, hidden_out, K);
-        if (rc) return rc;
-        T12_REQUIRE(!post_w || residual, "t12_gemv_glu: a post-norm weight without a residual");
-    }
-    GemvParams p;
-    p.seg[0] = two[0];
-    p.seg[1] = two[1];
-    p.nseg = 2;
-    p.K = K;
-    p.act = (const uint16_t*)act_bf16;
-    p.out_bf16 = (uint16_t*)out_bf16;
-    p.add = nullptr;
-    p.nx = x;
-    p.nres = residual;
-    p.npost = post_w;
-    p.nw = norm_w;
-    p.hidden_out = hidden_out;
-    p.eps = eps;
-    p.glu = *glu;
-    hipStream_t st = (hipStream_t)stream;
-    if (act_bf16) return launch_swiglu<0>(p, st);
-    return post_w ? launch_swiglu<3>(p, st) : residual ? launch_swiglu<2>(p, st) : launch_swiglu<1>(p, st);
 }
 
 // One activation row per slot, each multiplied with the tensors of the expert the routing gave the slot (a device

@@ -35,10 +35,13 @@ __device__ __forceinline__ uint32_t pack_bf16(float lo, float hi)
     return __builtin_bit_cast(uint32_t, __builtin_convertvector((f2){lo, hi}, t12_bf16x2));
 }
 
+// What the pieces of a position's row are turned by: eight positions next to each other all differ, and four within an aligned
+// four differ above the lowest bit (they read two pieces each at once).
+__device__ __forceinline__ int turn(int position) { return ((position << 1) & 6) | ((position >> 2) & 1); }
 // Where element e of a position's row lies within the row.
 __device__ __forceinline__ int place(const T12LatentAttn& a, int position, int e)
 {
-    return a.matrix ? ((e >> 3) ^ (position & 7)) * 8 + (e & 7) : e;
+    return a.matrix ? ((e >> 3) ^ turn(position)) * 8 + (e & 7) : e;
 }
 
 }  // namespace latent_attn

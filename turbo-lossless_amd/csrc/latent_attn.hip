@@ -6,7 +6,7 @@
 // first rank of them, and a token's cache is that one row.
 //
 // A step is three launches: the key projection of the queries (beside it, in workgroups of their own, the cache store and the
-// rotations), attention, the value projection with the gate.  All three run on the matrix cores for the sizes that have
+// rotations; a launch of its own in prompt passes), attention, the value projection with the gate.  All three run on the matrix cores for the sizes that have
 // instances; 32-bit states and other sizes take the general forms.
 
 #include <algorithm>
@@ -19,12 +19,13 @@ using namespace latent_attn;
 
 namespace {
 
-// ---- what a row stores and asks with, by one workgroup of 256 threads: the normed latent and the rotated key part into the cache; the
-// rotated parts of the queries, and zeros in the padding, into the query rows.
+// ---- what a row stores and asks with, by one workgroup of 256 threads: the normed latent and the rotated key part into the cache;
+// the rotated parts of the queries, and zeros in the padding, into the query rows.
 template <typename T>
 __device__ __forceinline__ void store_row(const LatentParams& p, int r)
 {
     __shared__ float red[4];
+    __shared__ float2 turned[64];                          // (cos, sin) of the row's angles, as many as there is room for
     const T12LatentAttn& a = p.a;
     const int tid = threadIdx.x, half = a.rot_dim / 2;
     const T12Row row = p.rows[r];
@@ -34,28 +35,32 @@ __device__ __forceinline__ void store_row(const LatentParams& p, int r)
     float ss = 0.0f;
     for (int i = tid; i < a.rank; i += 256) ss += c[i] * c[i];
     ss = t12_wave_sum(ss);
-    __syncthreads();                                       // red may still be read for the row before
+    __syncthreads();                                       // red and turned may still be read for the row before
     if ((tid & 63) == 0) red[tid >> 6] = ss;
+    auto angle = [&](int i) {
+        float2 t;
+        sincosf((float)row.position * a.freqs[i], &t.y, &t.x);
+        return t;
+    };
+    for (int i = tid; i < min(half, 64); i += 256) turned[i] = angle(i);
     __syncthreads();
     const float rn = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)a.rank + a.eps);
     for (int i = tid; i < a.rank; i += 256) cache[place(a, row.position, i)] = to_cache<T>(c[i] * rn * a.norm_w[i]);
     for (int i = tid; i < half; i += 256) {
-        float sn, cs;
-        sincosf((float)row.position * a.freqs[i], &sn, &cs);
+        const float2 t = i < 64 ? turned[i] : angle(i);
         const float u = c[a.rank + i], v = c[a.rank + half + i];
-        cache[place(a, row.position, a.rank_p + i)] = to_cache<T>(u * cs - v * sn);
-        cache[place(a, row.position, a.rank_p + half + i)] = to_cache<T>(v * cs + u * sn);
+        cache[place(a, row.position, a.rank_p + i)] = to_cache<T>(u * t.x - v * t.y);
+        cache[place(a, row.position, a.rank_p + half + i)] = to_cache<T>(v * t.x + u * t.y);
     }
     T* q = (T*)p.q + (size_t)r * a.heads * a.row_p;
     const int qd = a.dim + a.rot_dim;
     for (int i = tid; i < a.heads * half; i += 256) {
         const int h = i / half, e = i % half;
-        float sn, cs;
-        sincosf((float)row.position * a.freqs[e], &sn, &cs);
+        const float2 t = e < 64 ? turned[e] : angle(e);
         const float* y = x + a.q_off + h * qd + a.dim;
         const float u = y[e], v = y[half + e];
-        q[(size_t)h * a.row_p + a.rank_p + e] = to_cache<T>(u * cs - v * sn);
-        q[(size_t)h * a.row_p + a.rank_p + half + e] = to_cache<T>(v * cs + u * sn);
+        q[(size_t)h * a.row_p + a.rank_p + e] = to_cache<T>(u * t.x - v * t.y);
+        q[(size_t)h * a.row_p + a.rank_p + half + e] = to_cache<T>(v * t.x + u * t.y);
     }
     const int pad = a.row_p - a.rank - a.rot_dim, low = a.rank_p - a.rank;
     for (int i = tid; i < a.heads * pad; i += 256) {
@@ -100,10 +105,14 @@ struct FromRows {                          // mean latents [row][head][rank_p]
     const T* x;
     int heads, head_ld;
     __device__ __forceinline__ float at(int r, int h, int k) const { return from_cache(x[((size_t)r * heads + h) * head_ld + k]); }
+    // (bf16 rows are padded: eight elements are always there)
     __device__ __forceinline__ void at8(int r, int h, int k, int left, float (&v)[8]) const
     {
+        const uint4 w = *(const uint4*)(x + ((size_t)r * heads + h) * head_ld + k);
+        const uint32_t u[4] = {w.x, w.y, w.z, w.w};
 #pragma unroll
-        for (int e = 0; e < 8; e++) v[e] = e < left ? at(r, h, k + e) : 0.0f;
+        for (int e = 0; e < 8; e++)
+            v[e] = e < left ? __builtin_bit_cast(float, e & 1 ? u[e >> 1] & 0xFFFF0000u : u[e >> 1] << 16) : 0.0f;
     }
 };
 struct FromParts {                         // sums of stretches of keys, put together here
@@ -127,16 +136,34 @@ struct FromParts {                         // sums of stretches of keys, put tog
         const size_t unit = (size_t)r * heads + h;
         const float2* q = parts + unit * splits;
         const float* x = sums + unit * splits * head_ld + k;          // (rows are padded: eight elements are always there)
-        float top = q[0].x, total = 0.0f;
-        for (int z = 1; z < splits; z++) top = fmaxf(top, q[z].x);
+        constexpr int G = 8;                                           // stretches whose loads are in flight together
+        float top = -1e30f, total = 0.0f;
+        for (int z0 = 0; z0 < splits; z0 += G) {
+            float2 w[G];
+#pragma unroll
+            for (int z = 0; z < G; z++) w[z] = q[min(z0 + z, splits - 1)];
+#pragma unroll
+            for (int z = 0; z < G; z++) top = fmaxf(top, w[z].x);
+        }
 #pragma unroll
         for (int e = 0; e < 8; e++) v[e] = 0.0f;
-        for (int z = 0; z < splits; z++) {
-            const float w = exp2f(q[z].x - top);
-            const t12_f32x4 a = *(const t12_f32x4*)(x + (size_t)z * head_ld), b = *(const t12_f32x4*)(x + (size_t)z * head_ld + 4);
-            total += w * q[z].y;
+        for (int z0 = 0; z0 < splits; z0 += G) {
+            float2 w[G];
+            t12_f32x4 a[G], b[G];
 #pragma unroll
-            for (int e = 0; e < 8; e++) v[e] += w * (e < 4 ? a[e & 3] : b[e & 3]);
+            for (int z = 0; z < G; z++) {
+                const int zz = min(z0 + z, splits - 1);
+                w[z] = q[zz];
+                a[z] = *(const t12_f32x4*)(x + (size_t)zz * head_ld);
+                b[z] = *(const t12_f32x4*)(x + (size_t)zz * head_ld + 4);
+            }
+#pragma unroll
+            for (int z = 0; z < G; z++) {
+                const float f = z0 + z < splits ? exp2f(w[z].x - top) : 0.0f;
+                total += f * w[z].y;
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] += f * (e < 4 ? a[z][e & 3] : b[z][e & 3]);
+            }
         }
         const float inv = 1.0f / total;
 #pragma unroll
@@ -198,39 +225,40 @@ struct ToGated {                           // times the head's sigmoid gate
     }
 };
 
-// ---- the product per head on the matrix cores: K a multiple of 32, base_exp in 0..240.  Workgroup = 64 outputs of a head for
-// 16 NT rows, a wave sixteen outputs; a lane takes 32 consecutive columns of one weight row per 128-column block (two sign/mantissa
-// pieces, one of nibbles), which feed four MFMAs with the activations in the same order.  The accumulators start from the
-// escapes' corrections.  STORE: workgroups with blockIdx.y == heads store the rows of their tile (latent attention's cache) instead.
+// ---- the product per head on the matrix cores: K a multiple of 32, base_exp in 0..240.  A workgroup has 16 NT rows of a head and a
+// stretch of its outputs, 64 at a time, a wave sixteen of them; a lane takes 32 consecutive columns of one weight row per
+// 128-column block (two sign/mantissa pieces, one of nibbles), which feed four MFMAs with the activations in the same order.  The
+// accumulators start from the escapes' corrections.  STORE: the workgroups with blockIdx.y == 0 store the rows of their tile (latent
+// attention's cache) instead.
 // Dynamic LDS: activations, 16-byte units of eight columns (paired like the decoded weights) [unit][16 NT rows].
 template <int NT, bool STORE, typename IN, typename OUT>
-__global__ __launch_bounds__(256) void heads_matrix_kernel(T12Segment w, int heads, int M, int K, IN in, OUT out, int n, const LatentParams lp)
+__global__ __launch_bounds__(256) void heads_matrix_kernel(T12Segment w, int M, int K, IN in, OUT out, int n, const LatentParams lp)
 {
     extern __shared__ uint4 lds[];
     constexpr int ROWS = 16 * NT;
-    const int r0 = blockIdx.x * ROWS, h = blockIdx.y, tid = threadIdx.x;
-    if (STORE && h == heads) {
+    const int r0 = blockIdx.x * ROWS, h = (int)blockIdx.y - (STORE ? 1 : 0), tid = threadIdx.x;
+    if (STORE && h < 0) {
         for (int r = r0 + blockIdx.z; r < min(r0 + ROWS, n); r += gridDim.z) store_row<uint16_t>(lp, r);
         return;
     }
     const int lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l = lane & 15, g4 = lane >> 4;
-    const int m0 = blockIdx.z * 64 + wave * 16, blocks = (K + 127) / 128, units = blocks * 16;
-    const size_t row = (size_t)h * M + min(m0 + l, M - 1);
-    const uint8_t* sm = w.sm + row * K;
-    const uint8_t* gr = w.gr + row * K / 2;
+    const int blocks = (K + 127) / 128, units = blocks * 16, tiles = (M + 63) / 64;
+    const int per = (tiles + (int)gridDim.z - 1) / (int)gridDim.z, t0 = blockIdx.z * per, t1 = min(t0 + per, tiles);
+    if (t0 >= t1) return;
     const uint32_t be2 = t12_opaque(((uint32_t)w.base_exp << 7) | ((uint32_t)w.base_exp << 23));
     uint4 s0, s1, gg;
-    auto request = [&](int b) {                            // (columns past K: the row's first ones again, times zero)
+    auto request = [&](int t, int b) {                     // (columns past K: the row's first ones again, times zero)
+        const size_t row = ((size_t)h * M + min(t * 64 + wave * 16 + l, M - 1)) * K;
         const int k = b * 128 + 32 * g4, at = k < K ? k : 0;
-        s0 = *(const uint4*)(sm + at);
-        s1 = *(const uint4*)(sm + at + 16);
-        gg = *(const uint4*)(gr + at / 2);
+        s0 = *(const uint4*)(w.sm + row + at);
+        s1 = *(const uint4*)(w.sm + row + at + 16);
+        gg = *(const uint4*)(w.gr + (row + at) / 2);
     };
-    request(0);
+    request(t0, 0);
     for (int i = tid; i < units * ROWS; i += 256) {
         const int u = i % units, r = i / units;
         float v[8];
-        if (u * 8 < K) in.at8(min(r0 + r, n - 1), h, u * 8, K - u * 8, v);
+        if (u * 8 < K && r0 + r < n) in.at8(r0 + r, h, u * 8, K - u * 8, v);
         else {
 #pragma unroll
             for (int e = 0; e < 8; e++) v[e] = 0.0f;
@@ -238,44 +266,48 @@ __global__ __launch_bounds__(256) void heads_matrix_kernel(T12Segment w, int hea
         lds[u * ROWS + r] = make_uint4(pack_bf16(v[0], v[4]), pack_bf16(v[1], v[5]), pack_bf16(v[2], v[6]), pack_bf16(v[3], v[7]));
     }
     __syncthreads();
-    t12_f32x4 acc[NT];
+    for (int t = t0; t < t1; t++) {
+        const int m0 = t * 64 + wave * 16 + 4 * g4;        // this lane's four outputs
+        t12_f32x4 acc[NT];
 #pragma unroll
-    for (int t = 0; t < NT; t++) acc[t] = (t12_f32x4)(0.0f);
-    if (w.row_off) {
+        for (int c = 0; c < NT; c++) acc[c] = (t12_f32x4)(0.0f);
+        if (w.row_off) {
+            int from[5];
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int m = min(m0 + 4 * g4 + i, M - 1);
-            const size_t at = (size_t)h * M + m;
-            for (int q = w.row_off[at]; q < w.row_off[at + 1]; q++) {
-                const float delta = t12_bf16_to_f32((uint16_t)w.correct[q]) - t12_bf16_to_f32((uint16_t)w.wrong[q]);
-                const int k = w.cols[q], e = k & 7;
+            for (int i = 0; i < 5; i++) from[i] = w.row_off[(size_t)h * M + min(m0 + i, M)];
 #pragma unroll
-                for (int t = 0; t < NT; t++)
-                    acc[t][i] += delta * t12_bf16_to_f32(((const uint16_t*)(lds + (k >> 3) * ROWS + t * 16 + l))[(e & 3) * 2 + (e >> 2)]);
+            for (int i = 0; i < 4; i++)
+                for (int q = from[i]; q < from[i + 1]; q++) {
+                    const float delta = t12_bf16_to_f32((uint16_t)w.correct[q]) - t12_bf16_to_f32((uint16_t)w.wrong[q]);
+                    const int k = w.cols[q], e = k & 7;
+#pragma unroll
+                    for (int c = 0; c < NT; c++)
+                        acc[c][i] += delta * t12_bf16_to_f32(((const uint16_t*)(lds + (k >> 3) * ROWS + c * 16 + l))[(e & 3) * 2 + (e >> 2)]);
+                }
+        }
+        for (int b = 0; b < blocks; b++) {
+            const uint4 c0 = s0, c1 = s1, cg = gg;
+            if (b + 1 < blocks) request(t, b + 1);
+            else request(min(t + 1, t1 - 1), 0);
+            uint32_t d[4][4];
+            t12_decode8(c0.x, c0.y, cg.x, be2, d[0]);
+            t12_decode8(c0.z, c0.w, cg.y, be2, d[1]);
+            t12_decode8(c1.x, c1.y, cg.z, be2, d[2]);
+            t12_decode8(c1.z, c1.w, cg.w, be2, d[3]);
+#pragma unroll
+            for (int e = 0; e < 4; e++) {
+                const t12_bf16x8 a = __builtin_bit_cast(t12_bf16x8, make_uint4(d[e][0], d[e][1], d[e][2], d[e][3]));
+#pragma unroll
+                for (int c = 0; c < NT; c++)
+                    acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                        a, __builtin_bit_cast(t12_bf16x8, lds[(b * 16 + 4 * g4 + e) * ROWS + c * 16 + l]), acc[c], 0, 0, 0);
             }
         }
-    }
-    for (int b = 0; b < blocks; b++) {
-        const uint4 c0 = s0, c1 = s1, cg = gg;
-        request(min(b + 1, blocks - 1));
-        uint32_t d[4][4];
-        t12_decode8(c0.x, c0.y, cg.x, be2, d[0]);
-        t12_decode8(c0.z, c0.w, cg.y, be2, d[1]);
-        t12_decode8(c1.x, c1.y, cg.z, be2, d[2]);
-        t12_decode8(c1.z, c1.w, cg.w, be2, d[3]);
 #pragma unroll
-        for (int e = 0; e < 4; e++) {
-            const t12_bf16x8 a = __builtin_bit_cast(t12_bf16x8, make_uint4(d[e][0], d[e][1], d[e][2], d[e][3]));
-#pragma unroll
-            for (int t = 0; t < NT; t++)
-                acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                    a, __builtin_bit_cast(t12_bf16x8, lds[(b * 16 + 4 * g4 + e) * ROWS + t * 16 + l]), acc[t], 0, 0, 0);
+        for (int c = 0; c < NT; c++) {
+            const int r = r0 + c * 16 + l;
+            if (r < n && m0 < M) out.put4(r, h, m0, M - m0, acc[c]);
         }
-    }
-#pragma unroll
-    for (int t = 0; t < NT; t++) {
-        const int r = r0 + t * 16 + l, m = m0 + 4 * g4;
-        if (r < n && m < M) out.put4(r, h, m, M - m, acc[t]);
     }
 }
 
@@ -284,11 +316,15 @@ bool matrix_product(const T12Segment& w, int K) { return K % 32 == 0 && K <= 512
 template <bool STORE, typename IN, typename OUT>
 void launch_heads(const T12Segment& w, int M, int K, const IN& in, const OUT& out, const LatentParams& p, hipStream_t st)
 {
-    const int heads = p.a.heads, nt = p.n > 16 && (!STORE || K <= 384) ? 4 : 1, units = (K + 127) / 128 * 16;
-    const dim3 grid((p.n + 16 * nt - 1) / (16 * nt), heads + (STORE ? 1 : 0), (M + 63) / 64);
+    // rows per workgroup: 64 for prompt passes, 16 for decode steps; outputs in as few stretches as still give the chip two
+    // workgroups per CU (the activations of a tile are staged once per stretch)
+    const int heads = p.a.heads, nt = p.n > 128 ? 4 : 1, units = (K + 127) / 128 * 16, tiles = (M + 63) / 64;
+    const int groups = (p.n + 16 * nt - 1) / (16 * nt) * heads, stretches = std::min(tiles, (511 + groups) / groups);
+    const dim3 grid((p.n + 16 * nt - 1) / (16 * nt), heads + (STORE ? 1 : 0), stretches);
     const size_t lds = (size_t)units * 16 * nt * 16;
-    if (nt == 4) hipLaunchKernelGGL((heads_matrix_kernel<4, STORE, IN, OUT>), grid, dim3(256), lds, st, w, heads, M, K, in, out, p.n, p);
-    else hipLaunchKernelGGL((heads_matrix_kernel<1, STORE, IN, OUT>), grid, dim3(256), lds, st, w, heads, M, K, in, out, p.n, p);
+    if constexpr (STORE) hipLaunchKernelGGL((heads_matrix_kernel<1, true, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, p);
+    else if (nt == 4) hipLaunchKernelGGL((heads_matrix_kernel<4, false, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, p);
+    else hipLaunchKernelGGL((heads_matrix_kernel<1, false, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, p);
 }
 
 // ---- attention, general form: one workgroup per (row, head), any sizes, fp32 arithmetic.  Dynamic LDS: the query [row_p].
@@ -394,10 +430,10 @@ __global__ __launch_bounds__(CT * 128) void latent_matrix_kernel(const LatentPar
     // LDS offsets of this lane within a block: keys for the scores (two pieces, the rest by constants), turned reads (four)
     int ko[2], vo[4];
 #pragma unroll
-    for (int s = 0; s < 2; s++) ko[s] = n * ROWB + ((4 * s + g4) ^ (n & 7)) * 16;
+    for (int s = 0; s < 2; s++) ko[s] = n * ROWB + ((4 * s + g4) ^ turn(n)) * 16;
     const int vk = 4 * g4 + (n >> 2);                      // key of this lane's turned reads
 #pragma unroll
-    for (int e = 0; e < 4; e++) vo[e] = vk * ROWB + ((2 * e + ((n & 3) >> 1)) ^ (vk & 7)) * 16 + (n & 1) * 8;
+    for (int e = 0; e < 4; e++) vo[e] = vk * ROWB + ((2 * e + ((n & 3) >> 1)) ^ turn(vk)) * 16 + (n & 1) * 8;
     int buf = 0;
     for (int b = b0; b < b1; b += 2) {
         __builtin_amdgcn_s_waitcnt(0x0F70);                // vmcnt(0): the blocks have landed
@@ -529,16 +565,18 @@ int launch_fast(LatentParams p, int max_position, void* out, int out_ld, hipStre
     const T12LatentAttn& a = p.a;
     const FromProjection q = {p.in, p.ld, a.q_off, a.dim + a.rot_dim, true};
     const ToQuery<uint16_t> to = {(uint16_t*)p.q, a.heads, a.row_p};
-    if (matrix_product(*a.k_up, a.dim)) launch_heads<true>(*a.k_up, a.rank, a.dim, q, to, p, st);
+    const bool product = matrix_product(*a.k_up, a.dim);
+    if (product && p.n <= 16) launch_heads<true>(*a.k_up, a.rank, a.dim, q, to, p, st);
     else {
         hipLaunchKernelGGL(latent_store_kernel<uint16_t>, dim3(p.n), dim3(256), 0, st, p);
-        hipLaunchKernelGGL((heads_general_kernel<FromProjection, ToQuery<uint16_t>>), dim3(p.n, a.heads, (a.rank + 63) / 64), dim3(256), 0, st,
+        if (product) launch_heads<false>(*a.k_up, a.rank, a.dim, q, to, p, st);
+        else hipLaunchKernelGGL((heads_general_kernel<FromProjection, ToQuery<uint16_t>>), dim3(p.n, a.heads, (a.rank + 63) / 64), dim3(256), 0, st,
                            *a.k_up, a.heads, a.rank, a.dim, q, to, p.n);
     }
-    // stretches of keys: as many as it takes to give every CU a workgroup, each at least four blocks
+    // stretches of keys: as many as it takes to give every CU a workgroup, each at least the two blocks of one step
     const int columns = p.run ? p.n * a.heads : a.heads, ct = columns > 32 ? 4 : columns > 16 ? 2 : 1;
     const int groups = (columns + ct * 16 - 1) / (ct * 16) * (p.run ? 1 : p.n), blocks = max_position / BLK + 1;
-    p.splits = std::max(1, std::min({(256 + groups - 1) / groups, (blocks + 3) / 4, MAX_SPLITS, PART_UNITS / (p.n * a.heads)}));
+    p.splits = std::max(1, std::min({(256 + groups - 1) / groups, (blocks + 1) / 2, MAX_SPLITS, PART_UNITS / (p.n * a.heads)}));
     const bool parts = !p.run || p.splits > 1;
     if (!parts) p.parts = nullptr;
     const int rc = ct == 4 ? launch_matrix_rank<4>(p, columns, st) : ct == 2 ? launch_matrix_rank<2>(p, columns, st) : launch_matrix_rank<1>(p, columns, st);

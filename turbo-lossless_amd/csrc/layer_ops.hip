@@ -40,6 +40,37 @@ __global__ __launch_bounds__(256) void embed_norm_kernel(const uint16_t* __restr
     const bool known = t >= 0 && t < n_vocab;
     const uint16_t* row = table + (size_t)(known ? t : 0) * width;
     float ss = 0.0f;
+    if (width % 8 == 0 && width <= 8192 && ((uintptr_t)table | (uintptr_t)out | (uintptr_t)w) % 16 == 0) {
+        uint4 e[4];                                        // everything the thread needs, requested at once
+#pragma unroll
+        for (int q = 0; q < 4; q++) {
+            const int i = (threadIdx.x + q * 256) * 8;
+            e[q] = i < width ? *(const uint4*)(row + i) : make_uint4(0, 0, 0, 0);
+        }
+#pragma unroll
+        for (int q = 0; q < 4; q++)
+            for (uint32_t u : {e[q].x, e[q].y, e[q].z, e[q].w}) {
+                const float a = __builtin_bit_cast(float, u << 16), b = __builtin_bit_cast(float, u & 0xFFFF0000u);
+                ss += a * a + b * b;
+            }
+        const float rn = known ? 1.0f / sqrtf(block_sum(ss, red) / (float)width + eps) : 0.0f;
+#pragma unroll
+        for (int q = 0; q < 4; q++) {
+            const int i = (threadIdx.x + q * 256) * 8;
+            if (i >= width) continue;
+            const uint32_t u[4] = {e[q].x, e[q].y, e[q].z, e[q].w};
+#pragma unroll
+            for (int h = 0; h < 2; h++) {
+                const t12_f32x4 g = *(const t12_f32x4*)(w + i + 4 * h);
+                t12_f32x4 v;
+#pragma unroll
+                for (int k = 0; k < 4; k++)
+                    v[k] = __builtin_bit_cast(float, k & 1 ? u[2 * h + (k >> 1)] & 0xFFFF0000u : u[2 * h + (k >> 1)] << 16) * rn * g[k];
+                *(t12_f32x4*)(out + (size_t)blockIdx.x * width + i + 4 * h) = v;
+            }
+        }
+        return;
+    }
     for (int i = threadIdx.x; i < width; i += 256) {
         const float v = t12_bf16_to_f32(row[i]);
         ss += v * v;
@@ -70,21 +101,30 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(const PostNormParam
     __shared__ float red[16];
     const size_t r = blockIdx.x;
     const int step = blockDim.x * E;
-    float v[ITEMS][E];
+    float v[ITEMS][E], res[ITEMS][E], pw[ITEMS][E], nw[ITEMS][E];
+    auto fetch = [](float (&d)[E], const float* src) {
+        if (VEC) {
+            const t12_f32x4 a = *(const t12_f32x4*)src;
+#pragma unroll
+            for (int e = 0; e < E; e++) d[e] = a[e];
+        } else d[0] = *src;
+    };
     float ss = 0.0f;
 #pragma unroll
-    for (int q = 0; q < ITEMS; q++) {
+    for (int q = 0; q < ITEMS; q++) {                      // (everything is requested ahead of the first sum)
         const int i = threadIdx.x * E + q * step;
 #pragma unroll
         for (int e = 0; e < E; e++) v[q][e] = 0.0f;
         if (i < p.width) {
+            fetch(res[q], p.residual + r * p.width + i);
+            fetch(pw[q], p.post_w + i);
+            fetch(nw[q], p.norm_w + i);
             const float* src = p.y + r * p.ld + i;
             for (int z = 0; z < p.nsplit; z++) {
-                if (VEC) {
-                    const t12_f32x4 a = *(const t12_f32x4*)(src + z * p.split_stride);
+                float a[E];
+                fetch(a, src + z * p.split_stride);
 #pragma unroll
-                    for (int e = 0; e < E; e++) v[q][e] += a[e];
-                } else v[q][0] += src[z * p.split_stride];
+                for (int e = 0; e < E; e++) v[q][e] += a[e];
             }
 #pragma unroll
             for (int e = 0; e < E; e++) ss += v[q][e] * v[q][e];
@@ -93,28 +133,34 @@ __global__ __launch_bounds__(1024) void post_norm_add_kernel(const PostNormParam
     const float pn = 1.0f / sqrtf(block_sum(ss, red) / (float)p.width + p.eps);
     ss = 0.0f;
 #pragma unroll
-    for (int q = 0; q < ITEMS; q++) {
-        const int i = threadIdx.x * E + q * step;
-        if (i < p.width) {
+    for (int q = 0; q < ITEMS; q++)
+        if ((int)threadIdx.x * E + q * step < p.width) {
 #pragma unroll
             for (int e = 0; e < E; e++) {
-                v[q][e] = p.residual[r * p.width + i + e] + v[q][e] * pn * p.post_w[i + e];
+                v[q][e] = res[q][e] + v[q][e] * pn * pw[q][e];
                 ss += v[q][e] * v[q][e];
-                p.x_out[r * p.width + i + e] = v[q][e];
             }
         }
-    }
     const float rn = 1.0f / sqrtf(block_sum(ss, red) / (float)p.width + p.eps);
 #pragma unroll
     for (int q = 0; q < ITEMS; q++) {
         const int i = threadIdx.x * E + q * step;
-        if (i < p.width) {
+        if (i >= p.width) continue;
+        float* x = p.x_out + r * p.width + i;
+        if constexpr (VEC) {
+            *(t12_f32x4*)x = (t12_f32x4){v[q][0], v[q][1], v[q][2], v[q][3]};
+            t12_f32x4 h;
 #pragma unroll
-            for (int e = 0; e < E; e++) {
-                const float h = v[q][e] * rn * p.norm_w[i + e];
-                if (F32) ((float*)p.h)[r * p.width + i + e] = h;
-                else ((uint16_t*)p.h)[r * p.width + i + e] = t12_f32_to_bf16(h);
-            }
+            for (int e = 0; e < 4; e++) h[e] = v[q][e] * rn * nw[q][e];
+            if (F32) *(t12_f32x4*)((float*)p.h + r * p.width + i) = h;
+            else
+                *(uint2*)((uint16_t*)p.h + r * p.width + i) = make_uint2(t12_f32_to_bf16(h[0]) | ((uint32_t)t12_f32_to_bf16(h[1]) << 16),
+                                                                         t12_f32_to_bf16(h[2]) | ((uint32_t)t12_f32_to_bf16(h[3]) << 16));
+        } else {
+            *x = v[q][0];
+            const float h = v[q][0] * rn * nw[q][0];
+            if (F32) ((float*)p.h)[r * p.width + i] = h;
+            else ((uint16_t*)p.h)[r * p.width + i] = t12_f32_to_bf16(h);
         }
     }
 }
@@ -261,7 +307,7 @@ int t12_post_norm_add(const float* y, const T12GemmPartials* part, const float* 
                         post_w, norm_w, eps, x_out, h, width};
     hipStream_t st = (hipStream_t)stream;
     auto aligned = [](const void* q) { return (uintptr_t)q % 16 == 0; };
-    if (width % 4 == 0 && width <= 8192 && p.ld % 4 == 0 && p.split_stride % 4 == 0 && aligned(p.y) && aligned(x_out)) {
+    if (width % 4 == 0 && width <= 8192 && p.ld % 4 == 0 && p.split_stride % 4 == 0 && aligned(p.y) && aligned(x_out) && aligned(residual) && aligned(post_w) && aligned(norm_w) && aligned(h)) {
         const int threads = width <= 4096 ? (width / 4 + 63) / 64 * 64 : 1024;
         if (h_f32) hipLaunchKernelGGL((post_norm_add_kernel<true, true>), dim3(n), dim3(threads), 0, st, p);
         else hipLaunchKernelGGL((post_norm_add_kernel<false, true>), dim3(n), dim3(threads), 0, st, p);

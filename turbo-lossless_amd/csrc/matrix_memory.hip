@@ -72,17 +72,20 @@ __device__ __forceinline__ float row_sum16(float v)
     return v;
 }
 
-// ---- the gates of a run: one wave per head, 64 tokens at a time.  (F, M) = (sum of f, largest i + the f behind it) of a stretch
-// compose, so m of every token comes from a scan over the lanes.  Tokens past the end: f = 0, i = -1e30.
+// ---- the gates of a run: one workgroup per head, a wave per 64 tokens.  (F, M) = (sum of f, largest i + the f behind it) of a
+// stretch compose, so m of every token comes from a scan over a wave's lanes and one over the waves.  Tokens past the end: f = 0,
+// i = -1e30.
+constexpr int GATE_WAVES = 8;
 template <bool CHUNKED>
-__global__ __launch_bounds__(64) void memory_gates_kernel(const MemoryParams p)
+__global__ __launch_bounds__(GATE_WAVES * 64) void memory_gates_kernel(const MemoryParams p)
 {
-    const int head = blockIdx.x, lane = threadIdx.x;
+    __shared__ float2 total[GATE_WAVES];
+    const int head = blockIdx.x, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const T12Row row = p.rows[0];
     float m0 = row.position == 0 ? 0.0f : state_in(p.m, row)[maximum_at(p.m, head)];
     float4* gate = p.gate + (size_t)head * p.nch * CH;
-    for (int c = 0; c < p.nch; c++) {
-        const int t = c * CH + lane;
+    for (int c0 = 0; c0 < p.nch; c0 += GATE_WAVES) {
+        const int c = c0 + wave, t = c * CH + lane;
         const float* x = p.in + (size_t)min(t, p.n - 1) * p.ld;
         const bool live = t < p.n;
         const float i = live ? input_gate(p, x, head) : -1e30f, f = live ? forget_gate(p, x, head) : 0.0f;
@@ -95,18 +98,29 @@ __global__ __launch_bounds__(64) void memory_gates_kernel(const MemoryParams p)
                 F += F1;
             }
         }
-        const float m = fmaxf(F + m0, M);
-        float before = __shfl_up(m, 1, 64);
-        if (lane == 0) before = m0;
-        if (CHUNKED) {
-            gate[t] = make_float4(F, i, m, expf(-m));
-            if (lane == 0) p.start[head * (p.nch + 1) + c] = m0;
-        } else {
-            gate[t] = make_float4(expf(f + before - m), expf(i - m), expf(-m), 0.0f);
+        if (lane == 63) total[wave] = make_float2(F, M);
+        __syncthreads();
+        float mine = m0, next = m0;                        // m ahead of this wave's tokens, and behind all waves'
+#pragma unroll
+        for (int w = 0; w < GATE_WAVES; w++) {
+            if (w == wave) mine = next;
+            next = fmaxf(next + total[w].x, total[w].y);
         }
-        m0 = __shfl(m, 63, 64);
+        const float m = fmaxf(F + mine, M);
+        float before = __shfl_up(m, 1, 64);
+        if (lane == 0) before = mine;
+        if (c < p.nch) {
+            if (CHUNKED) {
+                gate[t] = make_float4(F, i, m, expf(-m));
+                if (lane == 0) p.start[head * (p.nch + 1) + c] = mine;
+            } else {
+                gate[t] = make_float4(expf(f + before - m), expf(i - m), expf(-m), 0.0f);
+            }
+        }
+        m0 = next;
+        __syncthreads();                                   // (total is written again)
     }
-    if (lane == 0) state_out(p.m, row)[maximum_at(p.m, head)] = m0;
+    if (threadIdx.x == 0) state_out(p.m, row)[maximum_at(p.m, head)] = m0;
 }
 
 // ---- exact: one wave = four columns of a head, lane l of a DPP row the key channels RL l .. RL l + RL - 1.
@@ -242,6 +256,16 @@ __device__ __forceinline__ void limbs8(const float (&v)[8], t12_bf16x8 (&l)[3])
     }
 }
 
+// Four consecutive projections with their bias, of which `left` exist (the others zero).
+__device__ __forceinline__ t12_f32x4 projected4(const MemoryParams& p, const float* x, int at, int left)
+{
+    if (left >= 4 && ((uintptr_t)(x + at) | (uintptr_t)(p.bias + at)) % 16 == 0) return *(const t12_f32x4*)(x + at) + *(const t12_f32x4*)(p.bias + at);
+    t12_f32x4 v;
+#pragma unroll
+    for (int e = 0; e < 4; e++) v[e] = e < left ? x[at + e] + p.bias[at + e] : 0.0f;
+    return v;
+}
+
 // Operands of a chunk.  blockIdx.z == 0: q, k^T and the decay-weighted scores; z > 0: 64 value channels of v^T.
 // Dynamic LDS: q and k [64][dc + 8] bf16.
 __global__ __launch_bounds__(256) void memory_prep_kernel(const MemoryParams p)
@@ -255,11 +279,18 @@ __global__ __launch_bounds__(256) void memory_prep_kernel(const MemoryParams p)
     if (blockIdx.z > 0) {
         uint16_t* tile = (uint16_t*)lds4;                  // [64 tokens][66]
         const int j0 = (blockIdx.z - 1) * 64;
-        for (int i = tid; i < CH * 64; i += 256) {
-            const int t = i >> 6, j = j0 + (i & 63), vc = m.v_off + head * m.vdim + min(j, m.vdim - 1);
-            float v = 0.0f;
-            if (t < nt && j <= m.vdim) v = j == m.vdim ? 1.0f : x0[(size_t)t * p.ld + vc] + p.bias[vc];
-            tile[t * 66 + (i & 63)] = t12_f32_to_bf16(v);
+#pragma unroll
+        for (int i = 0; i < 4; i++) {                      // (token, four channels)
+            const int t = (tid >> 4) + i * 16, j = j0 + (tid & 15) * 4;
+            t12_f32x4 v = (t12_f32x4)(0.0f);
+            if (t < nt) {
+                v = projected4(p, x0 + (size_t)t * p.ld, m.v_off + head * m.vdim + j, m.vdim - j);
+#pragma unroll
+                for (int e = 0; e < 4; e++)
+                    if (j + e == m.vdim) v[e] = 1.0f;
+            }
+            *(uint32_t*)(tile + t * 66 + (tid & 15) * 4) = pack_bf16(v[0], v[1]);
+            *(uint32_t*)(tile + t * 66 + (tid & 15) * 4 + 2) = pack_bf16(v[2], v[3]);
         }
         __syncthreads();
         for (int i = tid; i < 64 * 8; i += 256) {          // (channel, eight tokens)
@@ -274,15 +305,13 @@ __global__ __launch_bounds__(256) void memory_prep_kernel(const MemoryParams p)
     }
     const int DC = p.dc, pitch = DC + 8;
     uint16_t *qs = (uint16_t*)lds4, *ks = qs + CH * pitch;
+#pragma unroll 4
     for (int i = tid; i < CH * DC / 4; i += 256) {
         const int t = i / (DC / 4), d = i % (DC / 4) * 4;
-        float q[4], k[4];
-#pragma unroll
-        for (int e = 0; e < 4; e++) {
-            const int dd = head * m.dim + min(d + e, m.dim - 1);
-            const bool live = t < nt && d + e < m.dim;
-            q[e] = live ? x0[(size_t)t * p.ld + m.q_off + dd] + p.bias[m.q_off + dd] : 0.0f;
-            k[e] = live ? x0[(size_t)t * p.ld + m.k_off + dd] + p.bias[m.k_off + dd] : 0.0f;
+        t12_f32x4 q = (t12_f32x4)(0.0f), k = q;
+        if (t < nt) {
+            q = projected4(p, x0 + (size_t)t * p.ld, m.q_off + head * m.dim + d, m.dim - d);
+            k = projected4(p, x0 + (size_t)t * p.ld, m.k_off + head * m.dim + d, m.dim - d);
         }
         const uint2 qw = make_uint2(pack_bf16(q[0], q[1]), pack_bf16(q[2], q[3]));
         *(uint2*)(qs + t * pitch + d) = qw;
@@ -343,8 +372,8 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(const MemoryParams p)
     __shared__ float wtab[2][CH], etab[2][CH];
     const T12MatrixMemory& m = p.m;
     constexpr int DC = NS * 128;
-    const int head = blockIdx.y, tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int n = lane & 15, g4 = lane >> 4, j = blockIdx.x * 16 + n;
+    const int head = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int n = lane & 15, g4 = lane >> 4, j = blockIdx.y * 16 + n;
     const bool live = j <= m.vdim;
     const T12Row row = p.rows[0];
     const size_t column = ((size_t)head * (m.vdim + 1) + min(j, m.vdim)) * m.dim_p;
@@ -387,10 +416,8 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(const MemoryParams p)
                 f.a[z][k] = *(const t12_bf16x8*)(p.aw + ((unit * 3 + k) * CH + wave * 16 + n) * CH + z * 32 + 8 * g4);
         }
     };
-    Frags f;
-    load(f, 0);
-    for (int c = 0; c < p.nch; c++) {
-        Frags next;
+    // a chunk on f; the next one's operands are on their way meanwhile
+    auto chunk = [&](const Frags& f, Frags& next, int c) {
         load(next, min(c + 1, p.nch - 1));
         const int buf = c & 1;
         if (wave == 0) {
@@ -454,7 +481,12 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(const MemoryParams p)
 #pragma unroll
                     for (int u = 0; u < 2; u++) S[s][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.k[s][u][z], l[k], S[s][u], 0, 0, 0);
         }
-        f = next;
+    };
+    Frags even, odd;
+    load(even, 0);
+    for (int c = 0; c < p.nch; c += 2) {
+        chunk(even, odd, c);
+        if (c + 1 < p.nch) chunk(odd, even, c + 1);
     }
     if (!live) return;
 #pragma unroll
@@ -466,30 +498,65 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(const MemoryParams p)
         }
 }
 
-// ---- one wave per (row, head): normaliser, RMS over the head, plain weight, sigmoid gate.  run: floors lie by head.
-template <bool F32>
+// ---- normaliser, RMS over the head, plain weight, sigmoid gate: WAVES waves per (row, head), their values in registers.  run:
+// floors lie by head.
+template <bool F32, int WAVES>
 __global__ __launch_bounds__(256) void memory_out_kernel(const MemoryParams p, int run, int chunked)
 {
+    constexpr int KEEP = 8, LANES = WAVES * 64;
+    __shared__ float red[4];
     const T12MatrixMemory& m = p.m;
-    const int item = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
-    if (item >= p.n * m.heads) return;
-    const int r = item / m.heads, head = item % m.heads, V = m.vdim;
-    const float4 g = run ? p.gate[(size_t)head * p.nch * CH + r] : p.gate[item];
-    const float* o = p.o + (size_t)item * (V + 1);
+    const int item = blockIdx.x * (4 / WAVES) + (threadIdx.x >> 6) / WAVES, i0 = threadIdx.x % LANES;
+    const bool live = item < p.n * m.heads;
+    const int r = min(item, p.n * m.heads - 1) / m.heads, head = min(item, p.n * m.heads - 1) % m.heads, V = m.vdim;
+    const float4 g = run ? p.gate[(size_t)head * p.nch * CH + r] : p.gate[(size_t)r * m.heads + head];
+    const float* o = p.o + ((size_t)r * m.heads + head) * (V + 1);
+    const float* gates = p.in + (size_t)r * p.ld + m.g_off + head * V;
+    float v[KEEP], z[KEEP];
+#pragma unroll
+    for (int q = 0; q < KEEP; q++) {
+        const int i = min(i0 + q * LANES, V - 1);
+        v[q] = o[i];
+        z[q] = gates[i] + p.bias[m.g_off + head * V + i];
+    }
     const float inv = 1.0f / (fmaxf(fabsf(o[V]), chunked ? g.w : g.z) + m.den_eps);
     float ss = 0.0f;
-    for (int i = lane; i < V; i += 64) {
-        const float v = o[i] * inv;
-        ss += v * v;
+#pragma unroll
+    for (int q = 0; q < KEEP; q++) {
+        v[q] *= inv;
+        ss += i0 + q * LANES < V ? v[q] * v[q] : 0.0f;
     }
-    const float rn = 1.0f / sqrtf(t12_wave_sum(ss) / (float)V + m.out_eps);
-    for (int i = lane; i < V; i += 64) {
+    for (int i = i0 + KEEP * LANES; i < V; i += LANES) ss += o[i] * inv * (o[i] * inv);
+    ss = t12_wave_sum(ss);
+    if (WAVES > 1) {
+        if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+        __syncthreads();
+        ss = 0.0f;
+#pragma unroll
+        for (int w = 0; w < WAVES; w++) ss += red[(threadIdx.x >> 6) / WAVES * WAVES + w];
+    }
+    const float rn = 1.0f / sqrtf(ss / (float)V + m.out_eps);
+    auto put = [&](int i, float x, float gate) {
         const int hc = head * V + i;
-        const float gate = p.in[(size_t)r * p.ld + m.g_off + hc] + p.bias[m.g_off + hc];
-        const float v = o[i] * inv * rn * m.norm_w[hc] * t12_sigmoid(gate);
-        if (F32) ((float*)p.out)[(size_t)r * p.out_ld + hc] = v;
-        else ((uint16_t*)p.out)[(size_t)r * p.out_ld + hc] = t12_f32_to_bf16(v);
-    }
+        x *= rn * m.norm_w[hc] * t12_sigmoid(gate);
+        if (F32) ((float*)p.out)[(size_t)r * p.out_ld + hc] = x;
+        else ((uint16_t*)p.out)[(size_t)r * p.out_ld + hc] = t12_f32_to_bf16(x);
+    };
+    if (!live) return;
+#pragma unroll
+    for (int q = 0; q < KEEP; q++)
+        if (i0 + q * LANES < V) put(i0 + q * LANES, v[q], z[q]);
+    for (int i = i0 + KEEP * LANES; i < V; i += LANES) put(i, o[i] * inv, gates[i] + p.bias[m.g_off + head * V + i]);
+}
+
+template <bool F32>
+void launch_out(const MemoryParams& p, int run, int chunked, hipStream_t st)
+{
+    const int items = p.n * p.m.heads;
+    if (items >= 2048 || p.m.vdim <= 128)
+        hipLaunchKernelGGL((memory_out_kernel<F32, 1>), dim3((items + 3) / 4), dim3(256), 0, st, p, run, chunked);
+    else
+        hipLaunchKernelGGL((memory_out_kernel<F32, 4>), dim3(items), dim3(256), 0, st, p, run, chunked);
 }
 
 int chunk_channels(int dim) { return dim <= 128 ? 128 : dim <= 256 ? 256 : 512; }
@@ -572,7 +639,7 @@ int t12_matrix_memory(const T12MatrixMemory* m, const float* in, const float* bi
             default: launch_token<32>(p, st); break;
         }
     } else if (exact) {
-        hipLaunchKernelGGL(memory_gates_kernel<false>, dim3(m->heads), dim3(64), 0, st, p);
+        hipLaunchKernelGGL(memory_gates_kernel<false>, dim3(m->heads), dim3(GATE_WAVES * 64), 0, st, p);
         const dim3 grid(m->heads, (cols + 3) / 4);
         switch (m->dim_p) {
             case 64: hipLaunchKernelGGL(memory_exact_kernel<4>, grid, dim3(64), 0, st, p); break;
@@ -581,7 +648,7 @@ int t12_matrix_memory(const T12MatrixMemory* m, const float* in, const float* bi
             default: hipLaunchKernelGGL(memory_exact_kernel<32>, grid, dim3(64), 0, st, p); break;
         }
     } else {
-        hipLaunchKernelGGL(memory_gates_kernel<true>, dim3(m->heads), dim3(64), 0, st, p);
+        hipLaunchKernelGGL(memory_gates_kernel<true>, dim3(m->heads), dim3(GATE_WAVES * 64), 0, st, p);
         const size_t lds = (size_t)2 * CH * (p.dc + 8) * 2;
         if (lds > 64 * 1024) {
             static std::once_flag once[16];                // the attribute is per device
@@ -597,7 +664,8 @@ int t12_matrix_memory(const T12MatrixMemory* m, const float* in, const float* bi
             }
         }
         hipLaunchKernelGGL(memory_prep_kernel, dim3(p.nch, m->heads, 1 + (p.vp + 63) / 64), dim3(256), lds, st, p);
-        const dim3 grid(p.vp / 16, m->heads);
+        // (the head is the fast axis: workgroups go to the chip's XCDs in turn, so an XCD's L2 holds few heads' operands)
+        const dim3 grid(m->heads, p.vp / 16);
         switch (p.dc) {
             case 128: hipLaunchKernelGGL(memory_scan_kernel<1>, grid, dim3(256), 0, st, p); break;
             case 256: hipLaunchKernelGGL(memory_scan_kernel<2>, grid, dim3(256), 0, st, p); break;
@@ -605,9 +673,8 @@ int t12_matrix_memory(const T12MatrixMemory* m, const float* in, const float* bi
         }
     }
     T12_CHECK_LAUNCH("t12_matrix_memory");
-    const dim3 grid((unsigned)(((size_t)n * m->heads + 3) / 4));
-    if (out_f32) hipLaunchKernelGGL(memory_out_kernel<true>, grid, dim3(256), 0, st, p, run, run && !exact);
-    else hipLaunchKernelGGL(memory_out_kernel<false>, grid, dim3(256), 0, st, p, run, run && !exact);
+    if (out_f32) launch_out<true>(p, run, run && !exact, st);
+    else launch_out<false>(p, run, run && !exact, st);
     T12_CHECK_LAUNCH("t12_matrix_memory(out)");
     return T12_OK;
 }
