@@ -56,7 +56,7 @@ class Memory:
             setattr(m, name + "_off", at)
             self.off[name] = slice(at, at + n)
             at += n
-        self.ld = at + 3
+        self.ld = (at + 3) // 4 * 4 if dim % 4 == 0 else at + 3
         t12.check(t12.lib.t12_memory_plan(C.byref(m), rows))
         # what a region holds before position 0 must not matter, not even when it is no number
         self.state = torch.full((regions * 2 * m.state_elems,), float("nan"), device=dev())

@@ -379,26 +379,78 @@ __global__ __launch_bounds__(256) void latent_general_kernel(const LatentParams 
 //   S^T = K Q^T    keys = A rows from LDS, columns -- (row, head) pairs -- = B from registers; lane (n, g4) = (lane % 16,
 //                  lane / 16) receives keys 4 g4 .. 4 g4 + 3 of both 16-key halves of a block for column n;
 //   P              softmax in fp32 with a running maximum per column; the weights enter the product as two bf16 (16 bits);
-//   O^T += C^T P^T the lane's eight weights are its B operand as they are; A = the block's latents turned around by the LDS's
+//   O^T += C^T P^T the lane's weights are its B operand as they are; A = the block's latents turned around by the LDS's
 //                  transposing reads, four keys of one channel per read.
 //
-// Workgroup = CT x 2 waves on 16 CT columns: wave w has columns 16 (w % CT) ..., and of every two blocks the one w / CT.  Blocks
-// come into LDS as they lie in the cache (their pieces are already spread over the banks), the next two while two are worked on.
+// Workgroup = CT x 2 waves on 16 CT columns.  The two waves of a column tile take one block of keys each for the scores, tell each
+// other those, and take one half of the channels each for the sums over both blocks' keys.  Blocks come into LDS as they lie
+// in the cache (their pieces are already spread over the banks), the next two while two are worked on.
 // run: columns run over all (row, head) pairs of the sequence; else blockIdx.z is the row.  blockIdx.y: stretch of keys.
-// Dynamic LDS: 2 x 2 blocks.
+// Dynamic LDS: 2 x 2 blocks, then the scores [CT x 2][2][64] x 16 bytes.
 typedef __attribute__((ext_vector_type(4))) short s16x4;
-typedef __attribute__((address_space(3))) uint8_t lds_byte;
+struct Turned {                            // eight keys of one channel: a lane's A operand
+    s16x4 half[2];
+};
+
+// Transposing reads of N channel tiles, both key halves of a block.  Written out because the compiler puts a wait for all
+// outstanding copies into LDS ahead of the builtin: the next blocks could not be on their way.  The reads have landed when
+// the statement ends.
+template <int AT, int ROWB>
+__device__ __forceinline__ void read_turned(const uint32_t (&at)[4], Turned (&v)[4])
+{
+    asm volatile("ds_read_b64_tr_b16 %0, %8 offset:%12\n\t"
+                 "ds_read_b64_tr_b16 %1, %8 offset:%13\n\t"
+                 "ds_read_b64_tr_b16 %2, %9 offset:%12\n\t"
+                 "ds_read_b64_tr_b16 %3, %9 offset:%13\n\t"
+                 "ds_read_b64_tr_b16 %4, %10 offset:%12\n\t"
+                 "ds_read_b64_tr_b16 %5, %10 offset:%13\n\t"
+                 "ds_read_b64_tr_b16 %6, %11 offset:%12\n\t"
+                 "ds_read_b64_tr_b16 %7, %11 offset:%13\n\t"
+                 "s_waitcnt lgkmcnt(0)"
+                 : "=&v"(v[0].half[0]), "=&v"(v[0].half[1]), "=&v"(v[1].half[0]), "=&v"(v[1].half[1]), "=&v"(v[2].half[0]),
+                   "=&v"(v[2].half[1]), "=&v"(v[3].half[0]), "=&v"(v[3].half[1])
+                 : "v"(at[0]), "v"(at[1]), "v"(at[2]), "v"(at[3]), "n"(AT), "n"(AT + 16 * ROWB)
+                 : "memory");
+}
+template <int AT, int ROWB>
+__device__ __forceinline__ void read_turned(const uint32_t (&at)[2], Turned (&v)[2])
+{
+    asm volatile("ds_read_b64_tr_b16 %0, %4 offset:%6\n\t"
+                 "ds_read_b64_tr_b16 %1, %4 offset:%7\n\t"
+                 "ds_read_b64_tr_b16 %2, %5 offset:%6\n\t"
+                 "ds_read_b64_tr_b16 %3, %5 offset:%7\n\t"
+                 "s_waitcnt lgkmcnt(0)"
+                 : "=&v"(v[0].half[0]), "=&v"(v[0].half[1]), "=&v"(v[1].half[0]), "=&v"(v[1].half[1])
+                 : "v"(at[0]), "v"(at[1]), "n"(AT), "n"(AT + 16 * ROWB)
+                 : "memory");
+}
+
+// acc[e] += (channel tiles J, J + 1, ... of a block, N at a time) x both limbs of the weights
+template <int EH, int N, int ROWB, int J = 0>
+__device__ __forceinline__ void add_block(const uint32_t (&at)[N], t12_bf16x8 hi, t12_bf16x8 lo, t12_f32x4 (&acc)[EH])
+{
+    Turned v[N];
+    read_turned<J / 4 * 128, ROWB>(at, v);
+#pragma unroll
+    for (int e = 0; e < N; e++) acc[J + e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(t12_bf16x8, v[e]), hi, acc[J + e], 0, 0, 0);
+#pragma unroll
+    for (int e = 0; e < N; e++) acc[J + e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(t12_bf16x8, v[e]), lo, acc[J + e], 0, 0, 0);
+    if constexpr (J + N < EH) add_block<EH, N, ROWB, J + N>(at, hi, lo, acc);
+}
 
 template <int RP, int CT>
-__global__ __launch_bounds__(CT * 128) void latent_matrix_kernel(const LatentParams p)
+__global__ __launch_bounds__(CT * 128, 2) void latent_matrix_kernel(const LatentParams p)
 {
-    constexpr int DT = RP + 2, ET = RP * 2, ROWB = DT * 64, BLKB = BLK * ROWB, NW = CT * 2;
+    constexpr int DT = RP + 2, EH = RP, ROWB = DT * 64, BLKB = BLK * ROWB, NW = CT * 2, N = EH < 4 ? EH : 4;
     extern __shared__ uint4 lds4[];
     uint8_t* lds = (uint8_t*)lds4;
+    t12_f32x4* told = (t12_f32x4*)(lds + 4 * BLKB);
     const T12LatentAttn& a = p.a;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), n = lane & 15, g4 = lane >> 4;
     const int ct = wave % CT, ph = wave / CT;
-    const T12Row row = p.rows[p.run ? 0 : blockIdx.z];
+    T12Row row = p.rows[p.run ? 0 : blockIdx.z];           // (the same for the workgroup, which the compiler cannot know)
+    row.position = __builtin_amdgcn_readfirstlane(row.position);
+    row.slot = __builtin_amdgcn_readfirstlane(row.slot);
     const int ncol = p.run ? p.n * a.heads : a.heads, first = blockIdx.x * CT * 16, col = first + ct * 16 + n;
     const size_t unit = (p.run ? 0 : (size_t)blockIdx.z * a.heads) + min(col, ncol - 1);
     const int pos = row.position + (p.run ? min(col, ncol - 1) / a.heads : 0);
@@ -411,8 +463,8 @@ __global__ __launch_bounds__(CT * 128) void latent_matrix_kernel(const LatentPar
 #pragma unroll
         for (int i = 0; i < 2 * BLKB / 1024 / NW; i++) {
             const int piece = wave + i * NW, which = piece / (BLKB / 1024), at = piece % (BLKB / 1024) * 1024;
-            const uint8_t* src = cache + (size_t)min(b + which, blocks - 1) * BLKB + at + lane * 16;
-            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
+            const uint8_t* src = cache + (size_t)min(b + which, blocks - 1) * BLKB + at;
+            __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(src + lane * 16u),
                                              (__attribute__((address_space(3))) void*)(lds + (buf * 2 + which) * BLKB + at), 16, 0, 0);
         }
     };
@@ -422,18 +474,23 @@ __global__ __launch_bounds__(CT * 128) void latent_matrix_kernel(const LatentPar
     const uint16_t* q = (const uint16_t*)p.q + unit * a.row_p + 8 * g4;
 #pragma unroll
     for (int s = 0; s < DT; s++) Q[s] = *(const t12_bf16x8*)(q + s * 32);
-    t12_f32x4 acc[ET];
+    t12_f32x4 acc[EH];
 #pragma unroll
-    for (int e = 0; e < ET; e++) acc[e] = (t12_f32x4)(0.0f);
+    for (int e = 0; e < EH; e++) acc[e] = (t12_f32x4)(0.0f);
     float top = -1e30f, sum = 0.0f;
     const float scale = a.scale * 1.44269504088896341f;
-    // LDS offsets of this lane within a block: keys for the scores (two pieces, the rest by constants), turned reads (four)
-    int ko[2], vo[4];
+    // offsets of this lane within a block: keys for the scores (two pieces, the rest by constants), turned reads (N tiles)
+    int ko[2];
 #pragma unroll
     for (int s = 0; s < 2; s++) ko[s] = n * ROWB + ((4 * s + g4) ^ turn(n)) * 16;
     const int vk = 4 * g4 + (n >> 2);                      // key of this lane's turned reads
+    const uint32_t lds_base = (uint32_t)(uintptr_t)(__attribute__((address_space(3))) uint8_t*)lds;
+    uint32_t vo[N];
 #pragma unroll
-    for (int e = 0; e < 4; e++) vo[e] = vk * ROWB + ((2 * e + ((n & 3) >> 1)) ^ turn(vk)) * 16 + (n & 1) * 8;
+    for (int e = 0; e < N; e++) {
+        const int tile = ph * EH + e;
+        vo[e] = lds_base + vk * ROWB + (tile >> 2) * 128 + ((2 * (tile & 3) + ((n & 3) >> 1)) ^ turn(vk)) * 16 + (n & 1) * 8;
+    }
     int buf = 0;
     for (int b = b0; b < b1; b += 2) {
         __builtin_amdgcn_s_waitcnt(0x0F70);                // vmcnt(0): the blocks have landed
@@ -442,19 +499,44 @@ __global__ __launch_bounds__(CT * 128) void latent_matrix_kernel(const LatentPar
         const uint8_t* blk = lds + (buf * 2 + ph) * BLKB;
         t12_f32x4 S[2];
         S[0] = S[1] = (t12_f32x4)(0.0f);
+        constexpr int G = DT % 3 == 0 ? 3 : 2;             // steps whose keys are read together, one group ahead
+        t12_bf16x8 K[2][G][2];
+        auto keys = [&](int g) {
 #pragma unroll
-        for (int s = 0; s < DT; s++)
+            for (int s = 0; s < G; s++)
 #pragma unroll
-            for (int u = 0; u < 2; u++)
-                S[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*(const t12_bf16x8*)(blk + ko[s & 1] + (s >> 1) * 128 + u * 16 * ROWB), Q[s],
-                                                               S[u], 0, 0, 0);
+                for (int u = 0; u < 2; u++) K[g & 1][s][u] = *(const t12_bf16x8*)(blk + ko[(g * G + s) & 1] + ((g * G + s) >> 1) * 128 + u * 16 * ROWB);
+        };
+        keys(0);
+#pragma unroll
+        for (int g = 0; g < DT / G; g++) {
+            if (g + 1 < DT / G) keys(g + 1);
+            __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+            for (int s = 0; s < G; s++)
+#pragma unroll
+                for (int u = 0; u < 2; u++) S[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(K[g & 1][s][u], Q[g * G + s], S[u], 0, 0, 0);
+        }
         // keys past the column's position, and a whole block past the stretch, get no weight
         const int left = b + ph < b1 ? pos - (b + ph) * BLK - 4 * g4 : -1;
-        float w[8], best = top;
 #pragma unroll
-        for (int i = 0; i < 8; i++) {
-            w[i] = (i >> 2) * 16 + (i & 3) <= left ? S[i >> 2][i & 3] * scale : -INFINITY;
-            best = fmaxf(best, w[i]);
+        for (int u = 0; u < 2; u++) {
+#pragma unroll
+            for (int i = 0; i < 4; i++) S[u][i] = u * 16 + i <= left ? S[u][i] * scale : -INFINITY;
+            told[(wave * 2 + u) * 64 + lane] = S[u];
+        }
+        __syncthreads();
+        const int other = (wave + CT) % NW;
+        float w[2][8], best = top;
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            const t12_f32x4 theirs = told[(other * 2 + u) * 64 + lane];
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                w[0][u * 4 + i] = ph == 0 ? S[u][i] : theirs[i];
+                w[1][u * 4 + i] = ph == 0 ? theirs[i] : S[u][i];
+                best = fmaxf(best, fmaxf(S[u][i], theirs[i]));
+            }
         }
         best = fmaxf(best, __shfl_xor(best, 16, 64));
         best = fmaxf(best, __shfl_xor(best, 32, 64));
@@ -462,69 +544,49 @@ __global__ __launch_bounds__(CT * 128) void latent_matrix_kernel(const LatentPar
         const bool grew = __any(best > top);
         top = best;
         sum *= back;
-        uint32_t hi[4], lo[4];
+        t12_bf16x8 hi8[2], lo8[2];
 #pragma unroll
-        for (int i = 0; i < 8; i++) {
-            w[i] = __builtin_amdgcn_exp2f(w[i] - best);
-            sum += w[i];
-        }
+        for (int z = 0; z < 2; z++) {
+            uint32_t hi[4], lo[4];
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            hi[i] = pack_bf16(w[2 * i], w[2 * i + 1]);
-            lo[i] = pack_bf16(w[2 * i] - __builtin_bit_cast(float, hi[i] << 16), w[2 * i + 1] - __builtin_bit_cast(float, hi[i] & 0xFFFF0000u));
+            for (int i = 0; i < 8; i++) {
+                w[z][i] = __builtin_amdgcn_exp2f(w[z][i] - best);
+                sum += w[z][i];
+            }
+#pragma unroll
+            for (int i = 0; i < 4; i++) {
+                hi[i] = pack_bf16(w[z][2 * i], w[z][2 * i + 1]);
+                lo[i] = pack_bf16(w[z][2 * i] - __builtin_bit_cast(float, hi[i] << 16),
+                                  w[z][2 * i + 1] - __builtin_bit_cast(float, hi[i] & 0xFFFF0000u));
+            }
+            hi8[z] = __builtin_bit_cast(t12_bf16x8, make_uint4(hi[0], hi[1], hi[2], hi[3]));
+            lo8[z] = __builtin_bit_cast(t12_bf16x8, make_uint4(lo[0], lo[1], lo[2], lo[3]));
         }
-        const t12_bf16x8 ph8 = __builtin_bit_cast(t12_bf16x8, make_uint4(hi[0], hi[1], hi[2], hi[3]));
-        const t12_bf16x8 pl8 = __builtin_bit_cast(t12_bf16x8, make_uint4(lo[0], lo[1], lo[2], lo[3]));
         if (grew) {
 #pragma unroll
-            for (int e = 0; e < ET; e++) acc[e] *= back;
+            for (int e = 0; e < EH; e++) acc[e] *= back;
         }
 #pragma unroll
-        for (int e = 0; e < ET; e++) {
-            struct { s16x4 h[2]; } v;
+        for (int z = 0; z < 2; z++) {
+            uint32_t at[N];
 #pragma unroll
-            for (int u = 0; u < 2; u++)
-                v.h[u] = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                    (__attribute__((address_space(3))) s16x4*)(lds_byte*)(blk + vo[e & 3] + (e >> 2) * 128 + u * 16 * ROWB));
-            const t12_bf16x8 vv = __builtin_bit_cast(t12_bf16x8, v);
-            acc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, ph8, acc[e], 0, 0, 0);
-            acc[e] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vv, pl8, acc[e], 0, 0, 0);
+            for (int e = 0; e < N; e++) at[e] = vo[e] + (buf * 2 + z) * BLKB;
+            add_block<EH, N, ROWB>(at, hi8[z], lo8[z], acc);
         }
         buf ^= 1;
     }
-    // the two waves of a column tile, put together through LDS
     sum += __shfl_xor(sum, 16, 64);
     sum += __shfl_xor(sum, 32, 64);
-    __syncthreads();
-    float2* ml = (float2*)lds;                             // [NW][16]
-    if (g4 == 0) ml[wave * 16 + n] = make_float2(top, sum);
-    __syncthreads();
-    const float2 theirs = ml[(wave + CT) % NW * 16 + n];
-    const float both = fmaxf(top, theirs.x), mine = exp2f(top - both);
-    sum = sum * mine + theirs.y * exp2f(theirs.x - both);
-    const float inv = p.parts ? mine : mine / sum;
-    constexpr int EG = ET < 8 ? ET : 8;
-    t12_f32x4* red = (t12_f32x4*)(lds + 1024);             // [CT][EG][64]
+    if (col >= ncol) return;
+    const float inv = p.parts ? 1.0f : 1.0f / sum;
 #pragma unroll
-    for (int e0 = 0; e0 < ET; e0 += EG) {
-        __syncthreads();
-        if (ph == 1) {
-#pragma unroll
-            for (int e = 0; e < EG; e++) red[(ct * EG + e) * 64 + lane] = acc[e0 + e] * inv;
-        }
-        __syncthreads();
-        if (ph == 0) {
-#pragma unroll
-            for (int e = 0; e < EG; e++) {
-                const t12_f32x4 s = acc[e0 + e] * inv + red[(ct * EG + e) * 64 + lane];
-                const int c = (e0 + e) * 16 + 4 * g4;
-                if (col >= ncol) continue;
-                if (p.parts) *(t12_f32x4*)((float*)p.mean + (unit * p.splits + blockIdx.y) * a.rank_p + c) = s;
-                else *(uint2*)((uint16_t*)p.mean + unit * a.rank_p + c) = make_uint2(pack_bf16(s[0], s[1]), pack_bf16(s[2], s[3]));
-            }
-        }
+    for (int e = 0; e < EH; e++) {
+        const int c = (ph * EH + e) * 16 + 4 * g4;
+        const t12_f32x4 s = acc[e] * inv;
+        if (p.parts) *(t12_f32x4*)((float*)p.mean + (unit * p.splits + blockIdx.y) * a.rank_p + c) = s;
+        else *(uint2*)((uint16_t*)p.mean + unit * a.rank_p + c) = make_uint2(pack_bf16(s[0], s[1]), pack_bf16(s[2], s[3]));
     }
-    if (p.parts && ph == 0 && g4 == 0 && col < ncol) p.parts[unit * p.splits + blockIdx.y] = make_float2(both, sum);
+    if (p.parts && ph == 0 && g4 == 0) p.parts[unit * p.splits + blockIdx.y] = make_float2(top, sum);
 }
 
 constexpr int MAX_SPLITS = 32;
@@ -533,7 +595,7 @@ constexpr int PART_UNITS = 16384;          // (row, head, stretch) sums a pass k
 template <int RP, int CT>
 int launch_matrix(const LatentParams& p, int columns, hipStream_t st)
 {
-    constexpr size_t lds = (size_t)4 * BLK * (RP + 2) * 64;
+    constexpr size_t lds = (size_t)4 * BLK * (RP + 2) * 64 + CT * 4096;
     if (lds > 64 * 1024) {
         static std::once_flag once[16];                    // the attribute is per device
         int dev = 0;

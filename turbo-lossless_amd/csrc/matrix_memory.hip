@@ -6,7 +6,7 @@
 //   * one token per row (decode): sixteen lanes own a column, the state streams through once;
 //   * a run of tokens, exact: the same columns walked token by token in fp32;
 //   * a run of tokens by chunks of 64 on the matrix cores: inside a chunk the recurrence is a causal product
-//     (q k^T under the decays) v, across chunks a [dim, 16] strip of the state per workgroup is read out with q and
+//     (q k^T under the decays) v, across chunks a [dim, 32] strip of the state per workgroup is read out with q and
 //     advanced with k^T (w v).  q, k and v are bf16 there; everything in 32 bits -- state, decay-weighted scores, weighted values --
 //     enters a product as three bf16 limbs (24 bits), and is accumulated in fp32.
 
@@ -30,7 +30,7 @@ struct MemoryParams {
     float4* gate;                          // [heads][nch * CH]; by chunks: F (log decay from the chunk's start), i, m, e^-m
                                            // exact: decay, entry weight, e^-m
     float* start;                          // [heads][nch + 1]: m at the chunks' starts
-    uint16_t *qb, *kt, *vt, *aw;           // chunk form: q [64][DC] (value_slot order), k^T [DC][64], v^T [VP][64], scores [3][64][64]
+    uint16_t *qb, *kt, *vt, *aw;           // chunk form: q, k^T, v^T and scores of every chunk, in fragments (below)
     int dc, vp;
     float* o;                              // [n][heads][vdim + 1]
     void* out;
@@ -228,10 +228,13 @@ __global__ __launch_bounds__(256) void memory_token_kernel(const MemoryParams p)
 }
 
 // ---- by chunks ----------------------------------------------------------------------------------------------------
-// Place of a channel inside a block of 32: lane group g of the matrix cores takes channels 4 g .. 4 g + 3 of both halves, which
-// is how an accumulator tile of the state holds them.
-__device__ __forceinline__ int channel_slot(int d) { return (d & ~31) + ((d & 15) >> 2) * 8 + ((d >> 4) & 1) * 4 + (d & 3); }
-
+// Operands lie as the matrix cores take them: fragments of 64 lanes x eight bf16, lane (n, g) = (lane % 16, lane / 16), so that a wave
+// loads a fragment as one contiguous kilobyte.
+//   q       [token tile][32-channel step]       lane: token n of the tile, channels 4 g .. 4 g + 3 of both halves of the step -- the
+//                                               order in which an accumulator tile of the state holds them
+//   k^T     [16-channel tile][32-token half]    lane: channel n, tokens 8 g .. 8 g + 7
+//   v^T     [16-channel tile][32-token half]    the same
+//   scores  [token tile][32-token half][limb]   lane: query n of the tile, tokens 8 g .. 8 g + 7
 __device__ __forceinline__ uint32_t pack_bf16(float lo, float hi)
 {
     typedef __attribute__((ext_vector_type(2))) float f2;
@@ -256,18 +259,28 @@ __device__ __forceinline__ void limbs8(const float (&v)[8], t12_bf16x8 (&l)[3])
     }
 }
 
-// Four consecutive projections with their bias, of which `left` exist (the others zero).
-__device__ __forceinline__ t12_f32x4 projected4(const MemoryParams& p, const float* x, int at, int left)
+// Four consecutive projections with their bias, columns at .. at + 3 of which those below `end` exist (the others zero).  No branch:
+// the loads of an unrolled loop stay in flight together.
+template <bool WIDE>
+__device__ __forceinline__ t12_f32x4 projected4(const MemoryParams& p, const float* x, int at, int end)
 {
-    if (left >= 4 && ((uintptr_t)(x + at) | (uintptr_t)(p.bias + at)) % 16 == 0) return *(const t12_f32x4*)(x + at) + *(const t12_f32x4*)(p.bias + at);
     t12_f32x4 v;
+    if (WIDE) {                                            // everything aligned, sizes multiples of four
+        const int c = min(at, end - 4);
+        v = *(const t12_f32x4*)(x + c) + *(const t12_f32x4*)(p.bias + c);
+        return at < end ? v : (t12_f32x4)(0.0f);
+    }
 #pragma unroll
-    for (int e = 0; e < 4; e++) v[e] = e < left ? x[at + e] + p.bias[at + e] : 0.0f;
+    for (int e = 0; e < 4; e++) {
+        const int c = min(at + e, end - 1);
+        v[e] = at + e < end ? x[c] + p.bias[c] : 0.0f;
+    }
     return v;
 }
 
 // Operands of a chunk.  blockIdx.z == 0: q, k^T and the decay-weighted scores; z > 0: 64 value channels of v^T.
 // Dynamic LDS: q and k [64][dc + 8] bf16.
+template <bool WIDE>
 __global__ __launch_bounds__(256) void memory_prep_kernel(const MemoryParams p)
 {
     extern __shared__ uint4 lds4[];
@@ -278,53 +291,70 @@ __global__ __launch_bounds__(256) void memory_prep_kernel(const MemoryParams p)
     const float* x0 = p.in + (size_t)c * CH * p.ld;
     if (blockIdx.z > 0) {
         uint16_t* tile = (uint16_t*)lds4;                  // [64 tokens][66]
-        const int j0 = (blockIdx.z - 1) * 64;
+        const int j0 = (blockIdx.z - 1) * 64, from = m.v_off + head * m.vdim, jj = (tid & 15) * 4;
+        t12_f32x4 v[4];
 #pragma unroll
-        for (int i = 0; i < 4; i++) {                      // (token, four channels)
-            const int t = (tid >> 4) + i * 16, j = j0 + (tid & 15) * 4;
-            t12_f32x4 v = (t12_f32x4)(0.0f);
-            if (t < nt) {
-                v = projected4(p, x0 + (size_t)t * p.ld, m.v_off + head * m.vdim + j, m.vdim - j);
+        for (int i = 0; i < 4; i++)                        // (token, four channels)
+            v[i] = projected4<WIDE>(p, x0 + (size_t)min((tid >> 4) + i * 16, nt - 1) * p.ld, from + j0 + jj, from + m.vdim);
 #pragma unroll
-                for (int e = 0; e < 4; e++)
-                    if (j + e == m.vdim) v[e] = 1.0f;
-            }
-            *(uint32_t*)(tile + t * 66 + (tid & 15) * 4) = pack_bf16(v[0], v[1]);
-            *(uint32_t*)(tile + t * 66 + (tid & 15) * 4 + 2) = pack_bf16(v[2], v[3]);
+        for (int i = 0; i < 4; i++) {
+            const int t = (tid >> 4) + i * 16;
+#pragma unroll
+            for (int e = 0; e < 4; e++) v[i][e] = t >= nt ? 0.0f : j0 + jj + e == m.vdim ? 1.0f : v[i][e];
+            *(uint32_t*)(tile + t * 66 + jj) = pack_bf16(v[i][0], v[i][1]);
+            *(uint32_t*)(tile + t * 66 + jj + 2) = pack_bf16(v[i][2], v[i][3]);
         }
         __syncthreads();
-        for (int i = tid; i < 64 * 8; i += 256) {          // (channel, eight tokens)
-            const int jj = i >> 3, t8 = (i & 7) * 8;
-            if (j0 + jj >= p.vp) continue;
+        uint4* out = (uint4*)p.vt + unit * p.vp * CH / 8;
+        for (int i = tid; i < 64 * 8; i += 256) {          // (tile, half, lane)
+            const int n = i & 15, g = i >> 4 & 3, z = i >> 6 & 1, jt = i >> 7, ch = jt * 16 + n, t8 = z * 32 + g * 8;
+            if (j0 + ch >= p.vp) continue;
             uint32_t w[4];
 #pragma unroll
-            for (int e = 0; e < 4; e++) w[e] = tile[(t8 + 2 * e) * 66 + jj] | ((uint32_t)tile[(t8 + 2 * e + 1) * 66 + jj] << 16);
-            *(uint4*)(p.vt + (unit * p.vp + j0 + jj) * CH + t8) = make_uint4(w[0], w[1], w[2], w[3]);
+            for (int e = 0; e < 4; e++) w[e] = tile[(t8 + 2 * e) * 66 + ch] | ((uint32_t)tile[(t8 + 2 * e + 1) * 66 + ch] << 16);
+            out[((j0 / 16 + jt) * 2 + z) * 64 + (i & 63)] = make_uint4(w[0], w[1], w[2], w[3]);
         }
         return;
     }
-    const int DC = p.dc, pitch = DC + 8;
+    const int DC = p.dc, pitch = DC + 8, per_row = DC / 4;
     uint16_t *qs = (uint16_t*)lds4, *ks = qs + CH * pitch;
-#pragma unroll 4
-    for (int i = tid; i < CH * DC / 4; i += 256) {
-        const int t = i / (DC / 4), d = i % (DC / 4) * 4;
-        t12_f32x4 q = (t12_f32x4)(0.0f), k = q;
-        if (t < nt) {
-            q = projected4(p, x0 + (size_t)t * p.ld, m.q_off + head * m.dim + d, m.dim - d);
-            k = projected4(p, x0 + (size_t)t * p.ld, m.k_off + head * m.dim + d, m.dim - d);
+    const int qf = m.q_off + head * m.dim, kf = m.k_off + head * m.dim;
+    constexpr int U = 4;                                   // pieces whose loads are in flight together
+    for (int i0 = tid; i0 < CH * per_row; i0 += 256 * U) {
+        t12_f32x4 q[U], k[U];
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            const int i = i0 + u * 256, d = i % per_row * 4;
+            const float* x = x0 + (size_t)min(i / per_row, nt - 1) * p.ld;
+            q[u] = projected4<WIDE>(p, x, qf + d, qf + m.dim);
+            k[u] = projected4<WIDE>(p, x, kf + d, kf + m.dim);
         }
-        const uint2 qw = make_uint2(pack_bf16(q[0], q[1]), pack_bf16(q[2], q[3]));
-        *(uint2*)(qs + t * pitch + d) = qw;
-        *(uint2*)(ks + t * pitch + d) = make_uint2(pack_bf16(k[0], k[1]), pack_bf16(k[2], k[3]));
-        *(uint2*)(p.qb + (unit * CH + t) * DC + channel_slot(d)) = qw;
+#pragma unroll
+        for (int u = 0; u < U; u++) {
+            const int i = i0 + u * 256, t = i / per_row, d = i % per_row * 4;
+            const bool live = t < nt;
+            *(uint2*)(qs + t * pitch + d) = live ? make_uint2(pack_bf16(q[u][0], q[u][1]), pack_bf16(q[u][2], q[u][3])) : make_uint2(0, 0);
+            *(uint2*)(ks + t * pitch + d) = live ? make_uint2(pack_bf16(k[u][0], k[u][1]), pack_bf16(k[u][2], k[u][3])) : make_uint2(0, 0);
+        }
     }
     __syncthreads();
-    for (int i = tid; i < DC * 8; i += 256) {              // (channel, eight tokens)
-        const int d = i % DC, t8 = i / DC * 8;
-        uint32_t w[4];
+    {
+        uint4* out = (uint4*)p.qb + unit * DC * CH / 8;
+        const int steps = DC / 32;
+        for (int i = tid; i < steps * 4 * 64; i += 256) {
+            const int n = i & 15, g = i >> 4 & 3, f = i >> 6, step = f % steps, tile = f / steps;
+            const uint16_t* q = qs + (tile * 16 + n) * pitch + step * 32 + 4 * g;
+            const uint2 lo = *(const uint2*)q, hi = *(const uint2*)(q + 16);
+            out[i] = make_uint4(lo.x, lo.y, hi.x, hi.y);
+        }
+        out = (uint4*)p.kt + unit * DC * CH / 8;
+        for (int i = tid; i < DC / 16 * 2 * 64; i += 256) {
+            const int n = i & 15, g = i >> 4 & 3, z = i >> 6 & 1, d = (i >> 7) * 16 + n, t8 = z * 32 + g * 8;
+            uint32_t w[4];
 #pragma unroll
-        for (int e = 0; e < 4; e++) w[e] = ks[(t8 + 2 * e) * pitch + d] | ((uint32_t)ks[(t8 + 2 * e + 1) * pitch + d] << 16);
-        *(uint4*)(p.kt + (unit * DC + d) * CH + t8) = make_uint4(w[0], w[1], w[2], w[3]);
+            for (int e = 0; e < 4; e++) w[e] = ks[(t8 + 2 * e) * pitch + d] | ((uint32_t)ks[(t8 + 2 * e + 1) * pitch + d] << 16);
+            out[i] = make_uint4(w[0], w[1], w[2], w[3]);
+        }
     }
     // scores: a wave takes sixteen queries
     const int lane = tid & 63, wave = tid >> 6, n = lane & 15, g4 = lane >> 4;
@@ -357,37 +387,45 @@ __global__ __launch_bounds__(256) void memory_prep_kernel(const MemoryParams p)
 #pragma unroll
             for (int k = 0; k < 3; k++) {
                 const uint16_t b = t12_f32_to_bf16(v);
-                aw[(k * CH + t) * CH + u] = b;
+                aw[((((wave * 2 + (s >> 1)) * 3 + k) * 64 + ((s & 1) * 2 + (n >> 3)) * 16 + 4 * g4 + i) * 8) + (n & 7)] = b;
                 v -= t12_bf16_to_f32(b);
             }
         }
 }
 
-// The chunks one after the other for sixteen value channels of a head.  Wave w holds key channels 32 NS w .. 32 NS (w + 1) - 1 of
+// The chunks one after the other for 16 NJ value channels of a head.  Wave w holds key channels 32 NS w .. 32 NS (w + 1) - 1 of
 // the strip in its accumulators; what q reads out of the four parts is added up through LDS.
 template <int NS>
 __global__ __launch_bounds__(256) void memory_scan_kernel(const MemoryParams p)
 {
-    __shared__ t12_f32x4 red[2][4][4][64];
-    __shared__ float wtab[2][CH], etab[2][CH];
+    constexpr int DC = NS * 128, NJ = 2;
+    __shared__ t12_f32x4 red[4][4][NJ][64];
+    __shared__ float wtab[CH], etab[CH];
     const T12MatrixMemory& m = p.m;
-    constexpr int DC = NS * 128;
     const int head = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    const int n = lane & 15, g4 = lane >> 4, j = blockIdx.y * 16 + n;
-    const bool live = j <= m.vdim;
+    const int n = lane & 15, g4 = lane >> 4, tiles = p.vp / 16;
     const T12Row row = p.rows[0];
-    const size_t column = ((size_t)head * (m.vdim + 1) + min(j, m.vdim)) * m.dim_p;
-    t12_f32x4 S[NS][2];
+    int jt[NJ], j[NJ];                                     // (a strip past the last one works on that one and stores nothing)
+    bool live[NJ];
+    size_t column[NJ];
+    t12_f32x4 S[NJ][NS][2];
 #pragma unroll
-    for (int s = 0; s < NS; s++)
+    for (int c = 0; c < NJ; c++) {
+        jt[c] = min((int)blockIdx.y * NJ + c, tiles - 1);
+        j[c] = jt[c] * 16 + n;
+        live[c] = (int)blockIdx.y * NJ + c < tiles && j[c] <= m.vdim;
+        column[c] = ((size_t)head * (m.vdim + 1) + min(j[c], m.vdim)) * m.dim_p;
 #pragma unroll
-        for (int u = 0; u < 2; u++) {
-            const int d = (wave * NS + s) * 32 + 16 * u + 4 * g4;
-            S[s][u] = (t12_f32x4)(0.0f);
-            if (row.position != 0 && live && d < m.dim_p) S[s][u] = *(const t12_f32x4*)(state_in(m, row) + column + d);
-        }
+        for (int s = 0; s < NS; s++)
+#pragma unroll
+            for (int u = 0; u < 2; u++) {
+                const int d = (wave * NS + s) * 32 + 16 * u + 4 * g4;
+                S[c][s][u] = (t12_f32x4)(0.0f);
+                if (row.position != 0 && live[c] && d < m.dim_p) S[c][s][u] = *(const t12_f32x4*)(state_in(m, row) + column[c] + d);
+            }
+    }
     struct Frags {
-        t12_bf16x8 q[4][NS], k[NS][2][2], v[2], a[2][3];
+        t12_bf16x8 q[4][NS], k[NS][2][2], v[NJ][2], a[2][3];
         float4 gate, end;
         float start;
     };
@@ -397,89 +435,115 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(const MemoryParams p)
         f.gate = gate[lane];
         f.end = gate[CH - 1];
         f.start = p.start[head * (p.nch + 1) + c];
+        const t12_bf16x8* q = (const t12_bf16x8*)p.qb + unit * (DC * CH / 8) + lane;
+        const t12_bf16x8* k = (const t12_bf16x8*)p.kt + unit * (DC * CH / 8) + lane;
+        const t12_bf16x8* v = (const t12_bf16x8*)p.vt + unit * p.vp * (CH / 8) + lane;
+        const t12_bf16x8* a = (const t12_bf16x8*)p.aw + (unit * 4 + wave) * 6 * 64 + lane;
 #pragma unroll
         for (int s = 0; s < NS; s++) {
 #pragma unroll
-            for (int t = 0; t < 4; t++)
-                f.q[t][s] = *(const t12_bf16x8*)(p.qb + (unit * CH + t * 16 + n) * DC + (wave * NS + s) * 32 + 8 * g4);
+            for (int t = 0; t < 4; t++) f.q[t][s] = q[(t * (DC / 32) + wave * NS + s) * 64];
 #pragma unroll
             for (int u = 0; u < 2; u++)
 #pragma unroll
-                for (int z = 0; z < 2; z++)
-                    f.k[s][u][z] = *(const t12_bf16x8*)(p.kt + (unit * DC + (wave * NS + s) * 32 + 16 * u + n) * CH + z * 32 + 8 * g4);
+                for (int z = 0; z < 2; z++) f.k[s][u][z] = k[(((wave * NS + s) * 2 + u) * 2 + z) * 64];
         }
 #pragma unroll
         for (int z = 0; z < 2; z++) {
-            f.v[z] = *(const t12_bf16x8*)(p.vt + (unit * p.vp + j) * CH + z * 32 + 8 * g4);
 #pragma unroll
-            for (int k = 0; k < 3; k++)
-                f.a[z][k] = *(const t12_bf16x8*)(p.aw + ((unit * 3 + k) * CH + wave * 16 + n) * CH + z * 32 + 8 * g4);
+            for (int i = 0; i < NJ; i++) f.v[i][z] = v[(jt[i] * 2 + z) * 64];
+#pragma unroll
+            for (int l = 0; l < 3; l++) f.a[z][l] = a[(z * 3 + l) * 64];
         }
     };
     // a chunk on f; the next one's operands are on their way meanwhile
     auto chunk = [&](const Frags& f, Frags& next, int c) {
         load(next, min(c + 1, p.nch - 1));
-        const int buf = c & 1;
-        if (wave == 0) {
-            wtab[buf][lane] = expf(f.end.x - f.gate.x + f.gate.y - f.end.z);
-            etab[buf][lane] = expf(f.gate.x + f.start - f.gate.z) * m.q_scale;
-        }
         const float keep = expf(f.end.x + f.start - f.end.z);
         // what the queries read out of this wave's part of the old state
-        t12_f32x4 acc[4];
+        t12_f32x4 acc[4][NJ];
 #pragma unroll
-        for (int t = 0; t < 4; t++) acc[t] = (t12_f32x4)(0.0f);
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int i = 0; i < NJ; i++) acc[t][i] = (t12_f32x4)(0.0f);
 #pragma unroll
         for (int s = 0; s < NS; s++) {
-            float v[8];
+            t12_bf16x8 l[NJ][3];
 #pragma unroll
-            for (int e = 0; e < 8; e++) v[e] = S[s][e >> 2][e & 3];
-            t12_bf16x8 l[3];
-            limbs8(v, l);
+            for (int i = 0; i < NJ; i++) {
+                float v[8];
+#pragma unroll
+                for (int e = 0; e < 8; e++) v[e] = S[i][s][e >> 2][e & 3];
+                limbs8(v, l[i]);
+            }
 #pragma unroll
             for (int k = 2; k >= 0; k--)
 #pragma unroll
-                for (int t = 0; t < 4; t++) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.q[t][s], l[k], acc[t], 0, 0, 0);
-        }
+                for (int t = 0; t < 4; t++)
 #pragma unroll
-        for (int t = 0; t < 4; t++) red[buf][wave][t][lane] = acc[t];
+                    for (int i = 0; i < NJ; i++) acc[t][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.q[t][s], l[i][k], acc[t][i], 0, 0, 0);
+        }
         // this chunk's own tokens, sixteen queries per wave
-        t12_f32x4 own = (t12_f32x4)(0.0f);
+        t12_f32x4 own[NJ];
+#pragma unroll
+        for (int i = 0; i < NJ; i++) own[i] = (t12_f32x4)(0.0f);
 #pragma unroll
         for (int z = 0; z < 2; z++)
 #pragma unroll
-            for (int k = 2; k >= 0; k--) own = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.a[z][k], f.v[z], own, 0, 0, 0);
-        __syncthreads();                                   // (the other buffer was last read before the previous barrier)
-        t12_f32x4 sum = red[buf][0][wave][lane];
+            for (int k = 2; k >= 0; k--)
 #pragma unroll
-        for (int w = 1; w < 4; w++) sum += red[buf][w][wave][lane];
+                for (int i = 0; i < NJ; i++) own[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.a[z][k], f.v[i][z], own[i], 0, 0, 0);
+        __syncthreads();                                   // (what the last chunk left in LDS has been read)
+        if (wave == 0) {
+            wtab[lane] = expf(f.end.x - f.gate.x + f.gate.y - f.end.z);
+            etab[lane] = expf(f.gate.x + f.start - f.gate.z) * m.q_scale;
+        }
 #pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const int t = wave * 16 + 4 * g4 + i;
-            if (live && c * CH + t < p.n)
-                p.o[((size_t)(c * CH + t) * m.heads + head) * (m.vdim + 1) + j] = sum[i] * etab[buf][t] + own[i];
+        for (int t = 0; t < 4; t++)
+#pragma unroll
+            for (int i = 0; i < NJ; i++) red[wave][t][i][lane] = acc[t][i];
+        __syncthreads();
+        const t12_f32x4 e4 = *(const t12_f32x4*)(etab + wave * 16 + 4 * g4);
+#pragma unroll
+        for (int i = 0; i < NJ; i++) {
+            t12_f32x4 sum = red[0][wave][i][lane];
+#pragma unroll
+            for (int w = 1; w < 4; w++) sum += red[w][wave][i][lane];
+            float* o = p.o + ((size_t)(c * CH + wave * 16 + 4 * g4) * m.heads + head) * (m.vdim + 1) + j[i];
+#pragma unroll
+            for (int r = 0; r < 4; r++)
+                if (live[i] && c * CH + wave * 16 + 4 * g4 + r < p.n) o[(size_t)r * m.heads * (m.vdim + 1)] = sum[r] * e4[r] + own[i][r];
         }
         // the state behind the chunk
 #pragma unroll
-        for (int s = 0; s < NS; s++)
+        for (int i = 0; i < NJ; i++)
 #pragma unroll
-            for (int u = 0; u < 2; u++) S[s][u] *= keep;
+            for (int s = 0; s < NS; s++)
+#pragma unroll
+                for (int u = 0; u < 2; u++) S[i][s][u] *= keep;
 #pragma unroll
         for (int z = 0; z < 2; z++) {
-            float v[8];
-            const uint4 raw = __builtin_bit_cast(uint4, f.v[z]);
-            const uint32_t w4[4] = {raw.x, raw.y, raw.z, raw.w};
+            const t12_f32x4 w0 = *(const t12_f32x4*)(wtab + z * 32 + 8 * g4), w1 = *(const t12_f32x4*)(wtab + z * 32 + 8 * g4 + 4);
+            t12_bf16x8 l[NJ][3];
 #pragma unroll
-            for (int e = 0; e < 8; e++)
-                v[e] = __builtin_bit_cast(float, e & 1 ? w4[e >> 1] & 0xFFFF0000u : w4[e >> 1] << 16) * wtab[buf][z * 32 + 8 * g4 + e];
-            t12_bf16x8 l[3];
-            limbs8(v, l);
+            for (int i = 0; i < NJ; i++) {
+                const uint4 raw = __builtin_bit_cast(uint4, f.v[i][z]);
+                const uint32_t r4[4] = {raw.x, raw.y, raw.z, raw.w};
+                float v[8];
+#pragma unroll
+                for (int e = 0; e < 8; e++)
+                    v[e] = __builtin_bit_cast(float, e & 1 ? r4[e >> 1] & 0xFFFF0000u : r4[e >> 1] << 16) * (e < 4 ? w0[e & 3] : w1[e & 3]);
+                limbs8(v, l[i]);
+            }
 #pragma unroll
             for (int k = 2; k >= 0; k--)
 #pragma unroll
                 for (int s = 0; s < NS; s++)
 #pragma unroll
-                    for (int u = 0; u < 2; u++) S[s][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.k[s][u][z], l[k], S[s][u], 0, 0, 0);
+                    for (int u = 0; u < 2; u++)
+#pragma unroll
+                        for (int i = 0; i < NJ; i++)
+                            S[i][s][u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(f.k[s][u][z], l[i][k], S[i][s][u], 0, 0, 0);
         }
     };
     Frags even, odd;
@@ -488,14 +552,17 @@ __global__ __launch_bounds__(256) void memory_scan_kernel(const MemoryParams p)
         chunk(even, odd, c);
         if (c + 1 < p.nch) chunk(odd, even, c + 1);
     }
-    if (!live) return;
 #pragma unroll
-    for (int s = 0; s < NS; s++)
+    for (int i = 0; i < NJ; i++) {
+        if (!live[i]) continue;
 #pragma unroll
-        for (int u = 0; u < 2; u++) {
-            const int d = (wave * NS + s) * 32 + 16 * u + 4 * g4;
-            if (d < m.dim_p) *(t12_f32x4*)(state_out(m, row) + column + d) = S[s][u];
-        }
+        for (int s = 0; s < NS; s++)
+#pragma unroll
+            for (int u = 0; u < 2; u++) {
+                const int d = (wave * NS + s) * 32 + 16 * u + 4 * g4;
+                if (d < m.dim_p) *(t12_f32x4*)(state_out(m, row) + column[i] + d) = S[i][s][u];
+            }
+    }
 }
 
 // ---- normaliser, RMS over the head, plain weight, sigmoid gate: WAVES waves per (row, head), their values in registers.  run:
@@ -656,16 +723,21 @@ int t12_matrix_memory(const T12MatrixMemory* m, const float* in, const float* bi
             if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 16) dev = 0;
             hipError_t e = hipSuccess;
             std::call_once(once[dev], [&] {
-                e = hipFuncSetAttribute((const void*)memory_prep_kernel, hipFuncAttributeMaxDynamicSharedMemorySize, 2 * CH * (512 + 8) * 2);
+                for (const void* k : {(const void*)memory_prep_kernel<true>, (const void*)memory_prep_kernel<false>})
+                    if (e == hipSuccess) e = hipFuncSetAttribute(k, hipFuncAttributeMaxDynamicSharedMemorySize, 2 * CH * (512 + 8) * 2);
             });
             if (e != hipSuccess) {
                 t12_set_error("t12_matrix_memory: cannot reserve %zu bytes of LDS", lds);
                 return T12_ELAUNCH;
             }
         }
-        hipLaunchKernelGGL(memory_prep_kernel, dim3(p.nch, m->heads, 1 + (p.vp + 63) / 64), dim3(256), lds, st, p);
+        bool wide = ld % 4 == 0 && m->dim % 4 == 0 && m->vdim % 4 == 0 && ((uintptr_t)in | (uintptr_t)bias) % 16 == 0;
+        for (int off : {m->q_off, m->k_off, m->v_off}) wide = wide && off % 4 == 0;
+        const dim3 prep(p.nch, m->heads, 1 + (p.vp + 63) / 64);
+        if (wide) hipLaunchKernelGGL(memory_prep_kernel<true>, prep, dim3(256), lds, st, p);
+        else hipLaunchKernelGGL(memory_prep_kernel<false>, prep, dim3(256), lds, st, p);
         // (the head is the fast axis: workgroups go to the chip's XCDs in turn, so an XCD's L2 holds few heads' operands)
-        const dim3 grid(m->heads, p.vp / 16);
+        const dim3 grid(m->heads, (p.vp / 16 + 1) / 2);
         switch (p.dc) {
             case 128: hipLaunchKernelGGL(memory_scan_kernel<1>, grid, dim3(256), 0, st, p); break;
             case 256: hipLaunchKernelGGL(memory_scan_kernel<2>, grid, dim3(256), 0, st, p); break;
