@@ -19,6 +19,8 @@ using namespace latent_attn;
 
 namespace {
 
+constexpr int MAX_SPLITS = 32;             // stretches of keys a row's attention is cut into
+
 // ---- what a row stores and asks with, by one workgroup of 256 threads: the normed latent and the rotated key part into the cache;
 // the rotated parts of the queries, and zeros in the padding, into the query rows.
 template <typename T>
@@ -75,12 +77,76 @@ __global__ __launch_bounds__(256) void latent_store_kernel(const LatentParams p)
     store_row<T>(p, blockIdx.x);
 }
 
+// LDS slot of (unit of eight columns, row): rows are rotated by the unit, so that neighbouring units of a row (how activations are
+// written) and neighbouring rows of a unit (how they are read) lie on different banks.
+template <int ROWS>
+__device__ __forceinline__ int slot(int u, int r) { return u * ROWS + ((r + u) & (ROWS - 1)); }
+
+// Rows r0 ... of a head's activations into LDS; columns past K and rows past n are zero.  Sixteen threads share a row.
+__device__ __forceinline__ uint4 paired(const float (&v)[8])
+{
+    return make_uint4(pack_bf16(v[0], v[4]), pack_bf16(v[1], v[5]), pack_bf16(v[2], v[6]), pack_bf16(v[3], v[7]));
+}
+__device__ __forceinline__ uint4 masked(uint4 w, bool live)
+{
+    const uint32_t m = live ? ~0u : 0u;
+    return make_uint4(w.x & m, w.y & m, w.z & m, w.w & m);
+}
+template <int ROWS, typename IN>
+__device__ __forceinline__ void stage_rows(const IN& in, uint4* lds, int r0, int n, int h, int units, int K)
+{
+    for (int u = threadIdx.x & 15; u < units; u += 16)
+        for (int r = threadIdx.x >> 4; r < ROWS; r += 16) {
+            float v[8];
+            const bool live = u * 8 < K && r0 + r < n;
+            if (live) in.at8(r0 + r, h, u * 8, K - u * 8, v);
+            lds[slot<ROWS>(u, r)] = live ? paired(v) : make_uint4(0, 0, 0, 0);
+        }
+}
+
+// The same with the loads of U units in flight together: in.request(r, h, k) reads eight elements that exist, Raw::unpack gives them.
+template <int ROWS, int U, typename IN>
+__device__ __forceinline__ void stage_rows_ahead(const IN& in, uint4* lds, int r0, int n, int h, int units, int K)
+{
+    constexpr int RS = ROWS / 16;
+    for (int u0 = threadIdx.x & 15; u0 < units; u0 += 16 * U) {
+        typename IN::Raw raw[U][RS];
+#pragma unroll
+        for (int j = 0; j < U; j++)
+#pragma unroll
+            for (int i = 0; i < RS; i++)
+                raw[j][i] = in.request(min(r0 + ((int)threadIdx.x >> 4) + i * 16, n - 1), h, min((u0 + j * 16) * 8, K - 8));
+#pragma unroll
+        for (int j = 0; j < U; j++)
+#pragma unroll
+            for (int i = 0; i < RS; i++) {
+                const int u = u0 + j * 16, r = (threadIdx.x >> 4) + i * 16;
+                float v[8];
+                raw[j][i].unpack(v);
+                if (U == 1 || u < units) lds[slot<ROWS>(u, r)] = masked(paired(v), u * 8 < K && r0 + r < n);
+            }
+    }
+}
+
 // ---- a product per head: y[r, h, m] = sum_k W[h M + m, k] x[r, h, k].  General form: any sizes, one wave per sixteen outputs
 // of a (row, head); sums in fp32.
 struct FromProjection {                    // fp32 projections of the pass, rounded to what the state computes in
     const float* in;
     int ld, off, head_ld;
-    bool round;
+    bool round, wide;                      // wide: every vector is 16-byte aligned
+    struct Raw {
+        t12_f32x4 a, b;
+        __device__ __forceinline__ void unpack(float (&v)[8]) const
+        {
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] = e < 4 ? a[e & 3] : b[e & 3];
+        }
+    };
+    __device__ __forceinline__ Raw request(int r, int h, int k) const
+    {
+        const float* x = in + (size_t)r * ld + off + h * head_ld + k;
+        return {*(const t12_f32x4*)x, *(const t12_f32x4*)(x + 4)};
+    }
     __device__ __forceinline__ float at(int r, int h, int k) const
     {
         const float v = in[(size_t)r * ld + off + h * head_ld + k];
@@ -99,11 +165,27 @@ struct FromProjection {                    // fp32 projections of the pass, roun
 #pragma unroll
         for (int e = 0; e < 8; e++) v[e] = e < left ? x[e] : 0.0f;
     }
+    template <int ROWS>
+    __device__ __forceinline__ void stage(uint4* lds, int r0, int n, int h, int units, int K) const
+    {
+        if (wide) stage_rows_ahead<ROWS, 1>(*this, lds, r0, n, h, units, K);
+        else stage_rows<ROWS>(*this, lds, r0, n, h, units, K);
+    }
 };
 template <typename T>
 struct FromRows {                          // mean latents [row][head][rank_p]
     const T* x;
     int heads, head_ld;
+    struct Raw {
+        uint4 w;
+        __device__ __forceinline__ void unpack(float (&v)[8]) const
+        {
+            const uint32_t u[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] = __builtin_bit_cast(float, e & 1 ? u[e >> 1] & 0xFFFF0000u : u[e >> 1] << 16);
+        }
+    };
+    __device__ __forceinline__ Raw request(int r, int h, int k) const { return {*(const uint4*)(x + ((size_t)r * heads + h) * head_ld + k)}; }
     __device__ __forceinline__ float at(int r, int h, int k) const { return from_cache(x[((size_t)r * heads + h) * head_ld + k]); }
     // (bf16 rows are padded: eight elements are always there)
     __device__ __forceinline__ void at8(int r, int h, int k, int left, float (&v)[8]) const
@@ -113,6 +195,11 @@ struct FromRows {                          // mean latents [row][head][rank_p]
 #pragma unroll
         for (int e = 0; e < 8; e++)
             v[e] = e < left ? __builtin_bit_cast(float, e & 1 ? u[e >> 1] & 0xFFFF0000u : u[e >> 1] << 16) : 0.0f;
+    }
+    template <int ROWS>
+    __device__ __forceinline__ void stage(uint4* lds, int r0, int n, int h, int units, int K) const
+    {
+        stage_rows_ahead<ROWS, 2>(*this, lds, r0, n, h, units, K);
     }
 };
 struct FromParts {                         // sums of stretches of keys, put together here
@@ -169,7 +256,67 @@ struct FromParts {                         // sums of stretches of keys, put tog
 #pragma unroll
         for (int e = 0; e < 8; e++) v[e] = e < left ? v[e] * inv : 0.0f;
     }
+    template <int ROWS>
+    __device__ __forceinline__ void stage(uint4* lds, int r0, int n, int h, int units, int K) const
+    {
+        if (n > 1 || units > 64) {
+            stage_rows<ROWS>(*this, lds, r0, n, h, units, K);
+            return;
+        }
+        // a single row: the waves take the stretches in turn, and their sums are put together
+        __shared__ float share[4][64][8];
+        __shared__ float2 weight[4];
+        const int u = threadIdx.x & 63, wave = threadIdx.x >> 6;
+        const float2* q = parts + (size_t)h * splits;
+        const float* x = sums + (size_t)h * splits * head_ld + min(u * 8, head_ld - 8);
+        constexpr int G = 8;                               // all stretches there can be: 4 x G
+        float2 w[G];
+        t12_f32x4 a[G], b[G];
+#pragma unroll
+        for (int z = 0; z < G; z++) {
+            const int zz = min(wave + 4 * z, splits - 1);
+            w[z] = q[zz];
+            a[z] = *(const t12_f32x4*)(x + (size_t)zz * head_ld);
+            b[z] = *(const t12_f32x4*)(x + (size_t)zz * head_ld + 4);
+        }
+        float top = -1e30f, total = 0.0f, v[8];
+#pragma unroll
+        for (int z = 0; z < G; z++) top = fmaxf(top, w[z].x);
+#pragma unroll
+        for (int e = 0; e < 8; e++) v[e] = 0.0f;
+#pragma unroll
+        for (int z = 0; z < G; z++) {
+            const float f = wave + 4 * z < splits ? exp2f(w[z].x - top) : 0.0f;
+            total += f * w[z].y;
+#pragma unroll
+            for (int e = 0; e < 8; e++) v[e] += f * (e < 4 ? a[z][e & 3] : b[z][e & 3]);
+        }
+#pragma unroll
+        for (int e = 0; e < 8; e++) share[wave][u][e] = v[e];
+        if (u == 0) weight[wave] = make_float2(top, total);
+        __syncthreads();
+        for (int c = threadIdx.x & 15; c < units; c += 16) {
+            const int r = threadIdx.x >> 4;
+            float y[8], all = -1e30f, sum = 0.0f;
+#pragma unroll
+            for (int g = 0; g < 4; g++) all = fmaxf(all, weight[g].x);
+#pragma unroll
+            for (int e = 0; e < 8; e++) y[e] = 0.0f;
+#pragma unroll
+            for (int g = 0; g < 4; g++) {
+                const float f = exp2f(weight[g].x - all);
+                sum += f * weight[g].y;
+#pragma unroll
+                for (int e = 0; e < 8; e++) y[e] += f * share[g][c][e];
+            }
+            const float inv = 1.0f / sum;
+#pragma unroll
+            for (int e = 0; e < 8; e++) y[e] = c * 8 + e < K ? y[e] * inv : 0.0f;
+            for (int q = r; q < ROWS; q += 16) lds[slot<ROWS>(c, q)] = q == 0 ? paired(y) : make_uint4(0, 0, 0, 0);
+        }
+    }
 };
+static_assert(MAX_SPLITS <= 32, "a single row's stretches are taken by four waves, eight each");
 
 template <typename IN, typename OUT>
 __global__ __launch_bounds__(256) void heads_general_kernel(T12Segment w, int heads, int M, int K, IN in, OUT out, int n)
@@ -196,11 +343,13 @@ struct ToQuery {
     T* q;
     int heads, row_p;
     __device__ __forceinline__ void put(int r, int h, int m, float v) const { q[((size_t)r * heads + h) * row_p + m] = to_cache<T>(v); }
-    // four consecutive outputs (bf16), of which `left` exist
-    __device__ __forceinline__ void put4(int r, int h, int m, int left, t12_f32x4 v) const
+    __device__ __forceinline__ float factor(int, int) const { return 1.0f; }
+    // four consecutive outputs (bf16), of which `left` exist; wide: always all of them, at aligned places
+    __device__ __forceinline__ void put4(int r, int h, int m, int left, t12_f32x4 v, bool) const
     {
         T* o = q + ((size_t)r * heads + h) * row_p + m;
-        if (left >= 4) *(uint2*)o = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+        const uint2 w = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+        if (left >= 4) *(uint2*)o = w;
         else
             for (int e = 0; e < left; e++) o[e] = to_cache<T>(v[e]);
     }
@@ -215,98 +364,131 @@ struct ToGated {                           // times the head's sigmoid gate
     {
         out[(size_t)r * out_ld + h * vdim + m] = to_cache<T>(v * t12_sigmoid(in[(size_t)r * ld + g_off + h]));
     }
-    __device__ __forceinline__ void put4(int r, int h, int m, int left, t12_f32x4 v) const
+    __device__ __forceinline__ float factor(int r, int h) const { return t12_sigmoid(in[(size_t)r * ld + g_off + h]); }
+    __device__ __forceinline__ void put4(int r, int h, int m, int left, t12_f32x4 v, bool wide) const
     {
-        v *= t12_sigmoid(in[(size_t)r * ld + g_off + h]);
         T* o = out + (size_t)r * out_ld + h * vdim + m;
-        if (left >= 4 && (uintptr_t)o % 8 == 0) *(uint2*)o = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+        const uint2 w = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
+        if (wide) *(uint2*)o = w;
         else
             for (int e = 0; e < min(left, 4); e++) o[e] = to_cache<T>(v[e]);
     }
 };
 
 // ---- the product per head on the matrix cores: K a multiple of 32, base_exp in 0..240.  A workgroup has 16 NT rows of a head and a
-// stretch of its outputs, 64 at a time, a wave sixteen of them; a lane takes 32 consecutive columns of one weight row per
-// 128-column block (two sign/mantissa pieces, one of nibbles), which feed four MFMAs with the activations in the same order.  The
-// accumulators start from the escapes' corrections.  STORE: the workgroups with blockIdx.y == 0 store the rows of their tile (latent
-// attention's cache) instead.
-// Dynamic LDS: activations, 16-byte units of eight columns (paired like the decoded weights) [unit][16 NT rows].
-template <int NT, bool STORE, typename IN, typename OUT>
-__global__ __launch_bounds__(256) void heads_matrix_kernel(T12Segment w, int M, int K, IN in, OUT out, int n, const LatentParams lp)
+// stretch of its outputs, 64 MT at a time, a wave 16 MT of them; a lane takes 32 consecutive columns of MT weight rows per
+// 128-column block (two sign/mantissa pieces, one of nibbles), which feed four MFMAs each with the activations in the same order.
+// The accumulators start from the escapes' corrections, whose list for the workgroup's rows is brought into LDS ahead (a list or a
+// stretch too long for it is read where it lies).  STORE: the workgroups with blockIdx.y == 0 store the rows of their tile
+// (latent attention's cache) instead.
+// Dynamic LDS: activations, 16-byte units of eight columns (paired like the decoded weights), slot<16 NT>.
+template <int NT, int MT, bool STORE, typename IN, typename OUT>
+__global__ __launch_bounds__(256) void heads_matrix_kernel(T12Segment w, int M, int K, IN in, OUT out, int n, int wide, const LatentParams lp)
 {
     extern __shared__ uint4 lds[];
-    constexpr int ROWS = 16 * NT;
+    constexpr int ROWS = 16 * NT, LIST_ROWS = 512, LIST = 512;
+    __shared__ int list_row[LIST_ROWS + 1];                // first entry of every output row
+    __shared__ float2 list[LIST];                          // (column, correct - wrong)
     const int r0 = blockIdx.x * ROWS, h = (int)blockIdx.y - (STORE ? 1 : 0), tid = threadIdx.x;
     if (STORE && h < 0) {
         for (int r = r0 + blockIdx.z; r < min(r0 + ROWS, n); r += gridDim.z) store_row<uint16_t>(lp, r);
         return;
     }
     const int lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), l = lane & 15, g4 = lane >> 4;
-    const int blocks = (K + 127) / 128, units = blocks * 16, tiles = (M + 63) / 64;
+    const int blocks = (K + 127) / 128, units = blocks * 16, tiles = (M + 64 * MT - 1) / (64 * MT);
     const int per = (tiles + (int)gridDim.z - 1) / (int)gridDim.z, t0 = blockIdx.z * per, t1 = min(t0 + per, tiles);
     if (t0 >= t1) return;
     const uint32_t be2 = t12_opaque(((uint32_t)w.base_exp << 7) | ((uint32_t)w.base_exp << 23));
-    uint4 s0, s1, gg;
+    uint4 s0[MT], s1[MT], gg[MT];
     auto request = [&](int t, int b) {                     // (columns past K: the row's first ones again, times zero)
-        const size_t row = ((size_t)h * M + min(t * 64 + wave * 16 + l, M - 1)) * K;
         const int k = b * 128 + 32 * g4, at = k < K ? k : 0;
-        s0 = *(const uint4*)(w.sm + row + at);
-        s1 = *(const uint4*)(w.sm + row + at + 16);
-        gg = *(const uint4*)(w.gr + (row + at) / 2);
+#pragma unroll
+        for (int i = 0; i < MT; i++) {
+            const size_t row = ((size_t)h * M + min(((t * 4 + wave) * MT + i) * 16 + l, M - 1)) * K;
+            s0[i] = *(const uint4*)(w.sm + row + at);
+            s1[i] = *(const uint4*)(w.sm + row + at + 16);
+            gg[i] = *(const uint4*)(w.gr + (row + at) / 2);
+        }
     };
     request(t0, 0);
-    for (int i = tid; i < units * ROWS; i += 256) {
-        const int u = i % units, r = i / units;
-        float v[8];
-        if (u * 8 < K && r0 + r < n) in.at8(r0 + r, h, u * 8, K - u * 8, v);
-        else {
-#pragma unroll
-            for (int e = 0; e < 8; e++) v[e] = 0.0f;
+    const int out0 = t0 * 64 * MT, outs = min(M - out0, (t1 - t0) * 64 * MT);
+    bool listed = false;
+    if (w.row_off) {
+        const int* rows = w.row_off + (size_t)h * M + out0;
+        const int e0 = rows[0], e1 = rows[outs];
+        listed = outs <= LIST_ROWS && e1 - e0 <= LIST;
+        if (listed) {
+            for (int i = tid; i <= outs; i += 256) list_row[i] = rows[i] - e0;
+            for (int i = tid; i < e1 - e0; i += 256)
+                list[i] = make_float2(__builtin_bit_cast(float, w.cols[e0 + i]),
+                                      t12_bf16_to_f32((uint16_t)w.correct[e0 + i]) - t12_bf16_to_f32((uint16_t)w.wrong[e0 + i]));
         }
-        lds[u * ROWS + r] = make_uint4(pack_bf16(v[0], v[4]), pack_bf16(v[1], v[5]), pack_bf16(v[2], v[6]), pack_bf16(v[3], v[7]));
     }
+    float factor[NT];
+#pragma unroll
+    for (int c = 0; c < NT; c++) factor[c] = out.factor(min(r0 + c * 16 + l, n - 1), h);
+    in.template stage<ROWS>(lds, r0, n, h, units, K);
     __syncthreads();
+    auto correct = [&](float (&a)[NT], int k, float delta) {
+        const int e = k & 7;
+#pragma unroll
+        for (int c = 0; c < NT; c++)
+            a[c] += delta * t12_bf16_to_f32(((const uint16_t*)(lds + slot<ROWS>(k >> 3, c * 16 + l)))[(e & 3) * 2 + (e >> 2)]);
+    };
     for (int t = t0; t < t1; t++) {
-        const int m0 = t * 64 + wave * 16 + 4 * g4;        // this lane's four outputs
-        t12_f32x4 acc[NT];
+        const int m0 = (t * 4 + wave) * MT * 16 + 4 * g4;  // the first four of this lane's outputs
+        t12_f32x4 acc[MT][NT];
 #pragma unroll
-        for (int c = 0; c < NT; c++) acc[c] = (t12_f32x4)(0.0f);
+        for (int i = 0; i < MT; i++)
+#pragma unroll
+            for (int c = 0; c < NT; c++) acc[i][c] = (t12_f32x4)(0.0f);
         if (w.row_off) {
-            int from[5];
 #pragma unroll
-            for (int i = 0; i < 5; i++) from[i] = w.row_off[(size_t)h * M + min(m0 + i, M)];
+            for (int i = 0; i < MT; i++)
 #pragma unroll
-            for (int i = 0; i < 4; i++)
-                for (int q = from[i]; q < from[i + 1]; q++) {
-                    const float delta = t12_bf16_to_f32((uint16_t)w.correct[q]) - t12_bf16_to_f32((uint16_t)w.wrong[q]);
-                    const int k = w.cols[q], e = k & 7;
+                for (int r = 0; r < 4; r++) {
+                    const int m = m0 + i * 16 + r;
+                    float a[NT] = {};
+                    if (listed) {
+                        const int q0 = list_row[min(m - out0, outs)], q1 = list_row[min(m + 1 - out0, outs)];
+                        for (int q = q0; q < q1; q++) correct(a, __builtin_bit_cast(int, list[q].x), list[q].y);
+                    } else if (m < M) {
+                        const int* at = w.row_off + (size_t)h * M + m;
+                        for (int q = at[0]; q < at[1]; q++)
+                            correct(a, w.cols[q], t12_bf16_to_f32((uint16_t)w.correct[q]) - t12_bf16_to_f32((uint16_t)w.wrong[q]));
+                    }
 #pragma unroll
-                    for (int c = 0; c < NT; c++)
-                        acc[c][i] += delta * t12_bf16_to_f32(((const uint16_t*)(lds + (k >> 3) * ROWS + c * 16 + l))[(e & 3) * 2 + (e >> 2)]);
+                    for (int c = 0; c < NT; c++) acc[i][c][r] = a[c];
                 }
         }
         for (int b = 0; b < blocks; b++) {
-            const uint4 c0 = s0, c1 = s1, cg = gg;
+            uint32_t d[MT][4][4];
+#pragma unroll
+            for (int i = 0; i < MT; i++) {
+                t12_decode8(s0[i].x, s0[i].y, gg[i].x, be2, d[i][0]);
+                t12_decode8(s0[i].z, s0[i].w, gg[i].y, be2, d[i][1]);
+                t12_decode8(s1[i].x, s1[i].y, gg[i].z, be2, d[i][2]);
+                t12_decode8(s1[i].z, s1[i].w, gg[i].w, be2, d[i][3]);
+            }
             if (b + 1 < blocks) request(t, b + 1);
             else request(min(t + 1, t1 - 1), 0);
-            uint32_t d[4][4];
-            t12_decode8(c0.x, c0.y, cg.x, be2, d[0]);
-            t12_decode8(c0.z, c0.w, cg.y, be2, d[1]);
-            t12_decode8(c1.x, c1.y, cg.z, be2, d[2]);
-            t12_decode8(c1.z, c1.w, cg.w, be2, d[3]);
 #pragma unroll
-            for (int e = 0; e < 4; e++) {
-                const t12_bf16x8 a = __builtin_bit_cast(t12_bf16x8, make_uint4(d[e][0], d[e][1], d[e][2], d[e][3]));
+            for (int e = 0; e < 4; e++)
 #pragma unroll
-                for (int c = 0; c < NT; c++)
-                    acc[c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                        a, __builtin_bit_cast(t12_bf16x8, lds[(b * 16 + 4 * g4 + e) * ROWS + c * 16 + l]), acc[c], 0, 0, 0);
-            }
+                for (int c = 0; c < NT; c++) {
+                    const t12_bf16x8 x = __builtin_bit_cast(t12_bf16x8, lds[slot<ROWS>(b * 16 + 4 * g4 + e, c * 16 + l)]);
+#pragma unroll
+                    for (int i = 0; i < MT; i++)
+                        acc[i][c] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                            __builtin_bit_cast(t12_bf16x8, make_uint4(d[i][e][0], d[i][e][1], d[i][e][2], d[i][e][3])), x, acc[i][c], 0, 0, 0);
+                }
         }
 #pragma unroll
         for (int c = 0; c < NT; c++) {
             const int r = r0 + c * 16 + l;
-            if (r < n && m0 < M) out.put4(r, h, m0, M - m0, acc[c]);
+#pragma unroll
+            for (int i = 0; i < MT; i++)
+                if (r < n && m0 + i * 16 < M) out.put4(r, h, m0 + i * 16, M - m0 - i * 16, acc[i][c] * factor[c], wide);
         }
     }
 }
@@ -314,17 +496,26 @@ __global__ __launch_bounds__(256) void heads_matrix_kernel(T12Segment w, int M, 
 bool matrix_product(const T12Segment& w, int K) { return K % 32 == 0 && K <= 512 && w.base_exp >= 0 && w.base_exp <= 240 && (!w.row_off || w.wrong); }
 
 template <bool STORE, typename IN, typename OUT>
-void launch_heads(const T12Segment& w, int M, int K, const IN& in, const OUT& out, const LatentParams& p, hipStream_t st)
+void launch_heads(const T12Segment& w, int M, int K, const IN& in, const OUT& out, int wide, const LatentParams& p, hipStream_t st)
 {
-    // rows per workgroup: 64 for prompt passes, 16 for decode steps; outputs in as few stretches as still give the chip two
-    // workgroups per CU (the activations of a tile are staged once per stretch)
-    const int heads = p.a.heads, nt = p.n > 128 ? 4 : 1, units = (K + 127) / 128 * 16, tiles = (M + 63) / 64;
-    const int groups = (p.n + 16 * nt - 1) / (16 * nt) * heads, stretches = std::min(tiles, (511 + groups) / groups);
-    const dim3 grid((p.n + 16 * nt - 1) / (16 * nt), heads + (STORE ? 1 : 0), stretches);
-    const size_t lds = (size_t)units * 16 * nt * 16;
-    if constexpr (STORE) hipLaunchKernelGGL((heads_matrix_kernel<1, true, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, p);
-    else if (nt == 4) hipLaunchKernelGGL((heads_matrix_kernel<4, false, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, p);
-    else hipLaunchKernelGGL((heads_matrix_kernel<1, false, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, p);
+    // rows per workgroup: 64 for prompt passes, 16 for decode steps; outputs in as few stretches as still give the chip enough
+    // workgroups (the activations of a tile are staged once per stretch)
+    const int heads = p.a.heads, units = (K + 127) / 128 * 16;
+    const bool prompt = p.n > 128 && K <= 512;
+    const int rows = prompt ? 64 : 16, tiles = (M + (prompt ? 127 : 63)) / (prompt ? 128 : 64);
+    const int groups = (p.n + rows - 1) / rows * heads, stretches = std::min(tiles, ((prompt ? 511 : 255) + groups) / groups);
+    const dim3 grid((p.n + rows - 1) / rows, heads + (STORE ? 1 : 0), stretches);
+    const size_t lds = (size_t)units * rows * 16;
+    if constexpr (STORE) hipLaunchKernelGGL((heads_matrix_kernel<1, 1, true, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, wide, p);
+    else if (prompt) {
+        static std::once_flag once[16];                    // the attribute is per device
+        int dev = 0;
+        if (hipGetDevice(&dev) != hipSuccess || dev < 0 || dev >= 16) dev = 0;
+        std::call_once(once[dev], [&] {
+            (void)hipFuncSetAttribute((const void*)heads_matrix_kernel<4, 2, false, IN, OUT>, hipFuncAttributeMaxDynamicSharedMemorySize, 64 * 1024);
+        });
+        hipLaunchKernelGGL((heads_matrix_kernel<4, 2, false, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, wide, p);
+    } else hipLaunchKernelGGL((heads_matrix_kernel<1, 1, false, IN, OUT>), grid, dim3(256), lds, st, w, M, K, in, out, p.n, wide, p);
 }
 
 // ---- attention, general form: one workgroup per (row, head), any sizes, fp32 arithmetic.  Dynamic LDS: the query [row_p].
@@ -589,7 +780,6 @@ __global__ __launch_bounds__(CT * 128, 2) void latent_matrix_kernel(const Latent
     if (p.parts && ph == 0 && g4 == 0) p.parts[unit * p.splits + blockIdx.y] = make_float2(top, sum);
 }
 
-constexpr int MAX_SPLITS = 32;
 constexpr int PART_UNITS = 16384;          // (row, head, stretch) sums a pass keeps when it keeps more than one stretch
 
 template <int RP, int CT>
@@ -625,13 +815,15 @@ int launch_matrix_rank(const LatentParams& p, int columns, hipStream_t st)
 int launch_fast(LatentParams p, int max_position, void* out, int out_ld, hipStream_t st)
 {
     const T12LatentAttn& a = p.a;
-    const FromProjection q = {p.in, p.ld, a.q_off, a.dim + a.rot_dim, true};
+    const int qd = a.dim + a.rot_dim;
+    const bool wide = (p.ld | a.q_off | qd) % 4 == 0 && (uintptr_t)p.in % 16 == 0;
+    const FromProjection q = {p.in, p.ld, a.q_off, qd, true, wide};
     const ToQuery<uint16_t> to = {(uint16_t*)p.q, a.heads, a.row_p};
     const bool product = matrix_product(*a.k_up, a.dim);
-    if (product && p.n <= 16) launch_heads<true>(*a.k_up, a.rank, a.dim, q, to, p, st);
+    if (product && p.n <= 16) launch_heads<true>(*a.k_up, a.rank, a.dim, q, to, 1, p, st);
     else {
         hipLaunchKernelGGL(latent_store_kernel<uint16_t>, dim3(p.n), dim3(256), 0, st, p);
-        if (product) launch_heads<false>(*a.k_up, a.rank, a.dim, q, to, p, st);
+        if (product) launch_heads<false>(*a.k_up, a.rank, a.dim, q, to, 1, p, st);
         else hipLaunchKernelGGL((heads_general_kernel<FromProjection, ToQuery<uint16_t>>), dim3(p.n, a.heads, (a.rank + 63) / 64), dim3(256), 0, st,
                            *a.k_up, a.heads, a.rank, a.dim, q, to, p.n);
     }
@@ -644,17 +836,17 @@ int launch_fast(LatentParams p, int max_position, void* out, int out_ld, hipStre
     const int rc = ct == 4 ? launch_matrix_rank<4>(p, columns, st) : ct == 2 ? launch_matrix_rank<2>(p, columns, st) : launch_matrix_rank<1>(p, columns, st);
     if (rc) return rc;
     const ToGated<uint16_t> gated = {(uint16_t*)out, out_ld, a.vdim, p.in, p.ld, a.g_off};
-    const bool fast = matrix_product(*a.v_up, a.rank);
+    const bool fast = matrix_product(*a.v_up, a.rank), aligned = a.vdim % 4 == 0 && out_ld % 4 == 0 && (uintptr_t)out % 8 == 0;
     const dim3 general(p.n, a.heads, (a.vdim + 63) / 64);
     if (parts) {
         const FromParts mean = {(const float*)p.mean, p.parts, a.heads, a.rank_p, p.splits};
-        if (fast) launch_heads<false>(*a.v_up, a.vdim, a.rank, mean, gated, p, st);
+        if (fast) launch_heads<false>(*a.v_up, a.vdim, a.rank, mean, gated, aligned, p, st);
         else
             hipLaunchKernelGGL((heads_general_kernel<FromParts, ToGated<uint16_t>>), general, dim3(256), 0, st, *a.v_up, a.heads, a.vdim, a.rank,
                                mean, gated, p.n);
     } else {
         const FromRows<uint16_t> mean = {(const uint16_t*)p.mean, a.heads, a.rank_p};
-        if (fast) launch_heads<false>(*a.v_up, a.vdim, a.rank, mean, gated, p, st);
+        if (fast) launch_heads<false>(*a.v_up, a.vdim, a.rank, mean, gated, aligned, p, st);
         else
             hipLaunchKernelGGL((heads_general_kernel<FromRows<uint16_t>, ToGated<uint16_t>>), general, dim3(256), 0, st, *a.v_up, a.heads, a.vdim,
                                a.rank, mean, gated, p.n);
@@ -666,7 +858,7 @@ template <typename T>
 void launch_general(const LatentParams& p, void* out, int out_ld, hipStream_t st)
 {
     const T12LatentAttn& a = p.a;
-    const FromProjection q = {p.in, p.ld, a.q_off, a.dim + a.rot_dim, sizeof(T) == 2};
+    const FromProjection q = {p.in, p.ld, a.q_off, a.dim + a.rot_dim, sizeof(T) == 2, false};
     const ToQuery<T> to = {(T*)p.q, a.heads, a.row_p};
     hipLaunchKernelGGL((heads_general_kernel<FromProjection, ToQuery<T>>), dim3(p.n, a.heads, (a.rank + 63) / 64), dim3(256), 0, st, *a.k_up,
                        a.heads, a.rank, a.dim, q, to, p.n);
