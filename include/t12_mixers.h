@@ -89,6 +89,16 @@ int t12_gemm_glu(const struct T12Segment* gate, const struct T12Segment* up, con
 int t12_gemv_glu(const struct T12Segment* gate, const struct T12Segment* up, const T12Glu* glu, const void* act_bf16, int K,
                  void* out_bf16, void* stream);
 
+/* The decode-GEMV behind a sublayer whose output goes through a norm of its own, norms with one gain for all columns:
+ *     s = residual + rmsnorm(x) gain_post  (-> hidden_out when given; it may not alias x or residual),
+ *     activations = bf16(rmsnorm(s) gain),
+ * x, residual fp32 [K]; K % 16 == 0, K <= 8192, base_exp in 0..240.  t12_gemv_norm (t12_abi.h), and t12_gemv_glu, on these. */
+int t12_gemv_gain_norm(const struct T12Segment* segs, int nseg, const float* x, const float* residual, float gain_post, float gain,
+                       float eps, float* hidden_out, int K, void* stream);
+int t12_gemv_glu_gain_norm(const struct T12Segment* gate, const struct T12Segment* up, const T12Glu* glu, const float* x,
+                           const float* residual, float gain_post, float gain, float eps, float* hidden_out, int K, void* out_bf16,
+                           void* stream);
+
 /* ---- windowed attention with sigmoid weights -------------------------------------------------------------------
  * Query head h reads key/value head h / (heads / kv_heads).  The query at position i sees the key at j <= i when
  * i - j < window or j < keep_first, with weight sigmoid(scale * q.k + head_bias[h]); weights are not normalised.

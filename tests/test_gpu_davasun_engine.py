@@ -93,17 +93,36 @@ def test_whole_prompts_and_portions(t12, model, fp32):
             eng.close()
 
 
-def test_unfused_decode_agrees(t12, model, monkeypatch):
-    path, cfg, t = model
-    tok = ids(cfg, 60, 2)
-    want = do.forward(cfg, t, tok)
-    monkeypatch.setenv("TURBO_NO_FUSE", "1")
+def stepped(t12, path, cfg, tok):
+    """Logits of every step of a batch-1 state, one token at a time."""
     eng = t12.Engine.load(path)
     try:
-        got = np.concatenate([eng.prefill_logits(0, [x]) for x in tok])
-        assert off(cfg, t, tok, got, want) < 1
+        got = []
+        for x in tok:
+            eng.forward([x])
+            got.append(eng.logits(cfg["vocab"]).cpu().numpy()[0])
+        return np.stack(got)
     finally:
         eng.close()
+
+
+@pytest.mark.parametrize("fused", [True, False])
+def test_steps_of_one_sequence(t12, model, fused, monkeypatch):
+    path, cfg, t = model
+    tok = ids(cfg, 60, 2)
+    if not fused:
+        monkeypatch.setenv("TURBO_NO_FUSE", "1")
+    assert off(cfg, t, tok, stepped(t12, path, cfg, tok), do.forward(cfg, t, tok)) < 1
+
+
+def test_decode_with_a_large_vocabulary(t12, tmp_path):
+    """Its head reads an input normed by a kernel of its own; smaller ones norm it in the product's prologue."""
+    for tail in (mlstm(), latent(ff=0)):
+        cfg = config([latent(), tail], width=80, vocab=8200)
+        path = str(tmp_path / tail["type"])
+        t = write_checkpoint(path, cfg, tensors(cfg, 17))
+        tok = ids(cfg, 40, 7)
+        assert off(cfg, t, tok, stepped(t12, path, cfg, tok), do.forward(cfg, t, tok)) < 1
 
 
 def test_picked_places_equal_all_places(t12, model):

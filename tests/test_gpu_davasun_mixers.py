@@ -415,6 +415,25 @@ def test_gated_decode_gemv(t12, oracle, M, K):
     assert rel_err(host(out), do.clamped_glu(wa @ xv, wb @ xv, 0.8)) < 5e-3
 
 
+@pytest.mark.parametrize("M, K", [(96, 64), (130, 1024), (64, 2064), (1000, 4096), (40, 8192)])
+def test_decode_gemv_with_the_norms_around_a_sublayer(t12, oracle, M, K):
+    rng = np.random.default_rng(M * K)
+    (ta, wa), (tb, wb) = (packed(t12, oracle, rng.standard_normal((M, K)) / np.sqrt(K)) for _ in range(2))
+    y, res = rng.standard_normal(K), 2 * rng.standard_normal(K)
+    yd, rd, out, hid = up(y), up(res), torch.empty(M, device=dev()), torch.empty(K, device=dev())
+    lib, st = t12.lib, t12.current_stream()
+    s = res + do.norm_one_gain(y, 0.7, 1e-5)
+    h = do.norm_one_gain(s, 1.3, 1e-5)
+    seg = (t12.Segment * 1)(ta.segment(out))
+    t12.check(lib.t12_gemv_gain_norm(seg, 1, yd.data_ptr(), rd.data_ptr(), 0.7, 1.3, 1e-5, hid.data_ptr(), K, st))
+    assert rel_err(host(hid), s) < 2e-6 and rel_err(host(out), wa @ h) < 1e-2
+    o16, hid2 = torch.empty(M, dtype=torch.bfloat16, device=dev()), torch.empty(K, device=dev())
+    g, u, glu = ta.segment(None), tb.segment(None), t12.Glu(0.8, 1.702, 1.0)
+    t12.check(lib.t12_gemv_glu_gain_norm(C.byref(g), C.byref(u), C.byref(glu), yd.data_ptr(), rd.data_ptr(), 0.7, 1.3, 1e-5, hid2.data_ptr(), K,
+                                         o16.data_ptr(), st))
+    assert torch.equal(hid, hid2) and rel_err(host(o16), do.clamped_glu(wa @ h, wb @ h, 0.8)) < 2e-2
+
+
 @pytest.mark.parametrize("M, K, B", [(200, 128, 6), (12400, 128, 70), (12400, 64, 300), (300, 256, 100)])
 def test_gated_product_over_a_batch(t12, oracle, M, K, B):
     rng = np.random.default_rng(M + B)

@@ -219,6 +219,9 @@ _SIGS = {
     "t12_post_norm_add": (_i, [_vp, C.POINTER(GemmPartials), _vp, _vp, _vp, C.c_float, _vp, _vp, _i, _i, _i, _vp]),
     "t12_glu": (_i, [_vp, _vp, C.POINTER(Glu), _vp, _i, C.c_size_t, _vp]),
     "t12_gemm_glu": (_i, [C.POINTER(Segment), C.POINTER(Segment), C.POINTER(Glu), _vp, _i, _i, _i, _vp, _i, _vp]),
+    "t12_gemv_gain_norm": (_i, [C.POINTER(Segment), _i, _vp, _vp, C.c_float, C.c_float, C.c_float, _vp, _i, _vp]),
+    "t12_gemv_glu_gain_norm": (_i, [C.POINTER(Segment), C.POINTER(Segment), C.POINTER(Glu), _vp, _vp, C.c_float, C.c_float, C.c_float, _vp, _i,
+                                    _vp, _vp]),
     "t12_gemv_glu": (_i, [C.POINTER(Segment), C.POINTER(Segment), C.POINTER(Glu), _vp, _i, _vp, _vp]),
     "t12_memory_plan": (_i, [C.POINTER(MatrixMemory), _i]),
     "t12_matrix_memory": (_i, [C.POINTER(MatrixMemory), _vp, _vp, _i, _vp, _i, _i, _i, _vp, _vp, _i, _i, _vp]),

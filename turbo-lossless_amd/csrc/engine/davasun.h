@@ -49,6 +49,7 @@ struct Layer {
     LayerConfig c;
     float *norm1, *norm1b;               // the gain, once per coordinate
     float *norm2, *norm2b;               // (null without a feed-forward)
+    float gain1, gain1b, gain2, gain2b;  // the same gains, once
     CompressedWeight w_in;               // [in_rows, width]
     CompressedWeight w_out;              // [width, out_cols]
     float* in_bias;                      // MLSTM: [in_ld], gate biases, zeros elsewhere
@@ -63,6 +64,7 @@ struct Data {
     Config config;
     std::vector<Layer> layers;
     float* embed_norm = nullptr;         // [width]
+    float final_gain = 1.0f;             // the final norm's, times the logit scale
 };
 
 Data* data_of(const Model* m);

@@ -134,6 +134,7 @@ void empty_layers(const Config& c, Data& d)
     for (const LayerConfig& k : c.layers) {
         Layer L;
         L.c = k;
+        L.gain1 = L.gain1b = L.gain2 = L.gain2b = 1.0f;
         L.norm1 = L.norm1b = L.norm2 = L.norm2b = L.in_bias = L.o_norm = L.freqs = nullptr;
         for (CompressedWeight* w : {&L.w_in, &L.w_out, &L.k_up, &L.v_up, &L.gate, &L.up, &L.down}) clear_weight(*w);
         d.layers.push_back(L);
@@ -293,6 +294,24 @@ Model* new_model(const Config& c)
     return m;
 }
 
+// What is read back once from the loaded tensors.
+void derive(Model* m)
+{
+    auto first = [](const float* v) {
+        float g = 1.0f;
+        if (v && !gpu_ok(hipMemcpy(&g, v, sizeof g, hipMemcpyDeviceToHost), "norm gain")) engine_fail("reading a norm's gain failed");
+        return g;
+    };
+    Data* d = data_of(m);
+    d->final_gain = first(m->output_norm);
+    for (Layer& L : d->layers) {
+        L.gain1 = first(L.norm1);
+        L.gain1b = first(L.norm1b);
+        L.gain2 = first(L.norm2);
+        L.gain2b = first(L.norm2b);
+    }
+}
+
 Model* load(const std::string& dir)
 {
     Config c;
@@ -311,6 +330,7 @@ Model* load(const std::string& dir)
             release(m);
             return nullptr;
         }
+        derive(m);
     } catch (...) {
         release(m);
         throw;
@@ -363,6 +383,7 @@ Model* create_synthetic_davasun(const std::string& config_json, uint64_t seed, f
             if (!gpu_ok(hipMemcpy(dst, v.data(), v.size() * sizeof(float), hipMemcpyHostToDevice), "synthetic constants"))
                 engine_fail("synthetic constants failed");
         }
+        derive(m);
     } catch (...) {
         release(m);
         throw;

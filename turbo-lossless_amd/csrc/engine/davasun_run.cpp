@@ -34,10 +34,21 @@ struct State : RegionState {
     void* h = nullptr;                           // normed input of a sublayer: bf16 (fp32 in 32-bit states) [rows, width]
     void* mix = nullptr;                         // the mixer's output [rows, out_cols]
     void* act = nullptr;                         // feed-forward activations [rows, ff]
-    bool no_fuse = false;                        // debugging: no products with epilogues
+    bool no_fuse = false;                        // debugging: no products with prologues or epilogues
+    bool fused_b1 = false;                       // one sequence, bf16: norms in the prologues of the projections
 };
 
 State* state_of(const InferenceState* s) { return (State*)(StateCommon*)s->impl; }
+
+// Every tensor behind a norm can take the decode-GEMV with the norms in its prologue.
+bool fused_b1_eligible(const Model* model)
+{
+    const Data& d = *data_of(model);
+    if (!region_norm_width(d.config.width) || !exp_ok(model->output_proj)) return false;
+    for (const Layer& L : d.layers)
+        if (!exp_ok(L.w_in) || (L.c.ff && (!exp_ok(L.gate) || !exp_ok(L.up)))) return false;
+    return true;
+}
 
 T12MatrixMemory memory_of(const Layer& L, float eps)
 {
@@ -141,6 +152,7 @@ InferenceState* create(Model* model, const StateOptions& o)
     st->mix = st->own(R * mix * el);
     st->act = st->own(R * ff * el);
     st->no_fuse = region_no_fuse();
+    st->fused_b1 = !st->f32 && !st->no_fuse && o.batch_size == 1 && fused_b1_eligible(model);
     check_gpu(hipMalloc((void**)&s->hidden, R * c.width * 4), "hipMalloc");
     check_gpu(hipMalloc((void**)&s->hidden2, R * c.width * 4), "hipMalloc");
     printf("  Sequence regions: %d, %.3f GB, %d rows per pass\n", regions, need / 1e9, st->rows);
@@ -166,8 +178,7 @@ void mixer(State* st, const Run& r, int R, int run, int max_position, hipStream_
              "latent attention");
 }
 
-// cur += norm(w . act) with gain `post`, then h = norm(cur) with gain `next`: what ends a sublayer.  (One kernel for both norms also for
-// a single row: a decode-GEMV that rebuilt them in every workgroup's prologue would read more than its weights.)
+// cur += norm(w . act) with gain `post`, then h = norm(cur) with gain `next`: what ends a sublayer.
 void close_sublayer(const CompressedWeight& w, const void* act, int K, const float* post, const float* next, float eps, int R, State* st,
                     float*& cur, float*& other, hipStream_t q)
 {
@@ -205,9 +216,60 @@ void gated_up(State* st, const Layer& L, int n, int R, hipStream_t q)
     must(t12_glu(st->gate, st->up, &unit, st->act, st->f32, (size_t)R * ff, q), "gated unit");
 }
 
+// One row.  A sublayer's output waits in st->y: the prologue of the next projection puts it through its norm, adds it to the
+// residual and norms the sum.  mLSTM: projections, memory, its output, output projection; latent attention: projections, key
+// projection beside the cache store, attention, value projection, output projection; feed-forward: gate|up with the unit, down.
+void pass_b1_fused(InferenceState* s, int position)
+{
+    State* st = state_of(s);
+    const Data& d = *data_of(s->model);
+    const Config& c = d.config;
+    const int n = c.width;
+    hipStream_t q = s->stream;
+    must(t12_embed_norm(s->model->token_embd, c.vocab, s->d_tokens, d.embed_norm, c.eps, s->hidden, n, 1, q), "embedding");
+    float *cur = s->hidden, *other = s->hidden2;
+    bool waits = false;                                            // st->y goes through a norm of gain `post`
+    float post = 1.0f;
+    auto project = [&](T12Segment g, const float* norm, float gain) {
+        if (!waits) {
+            must(t12_gemv_norm(&g, 1, cur, nullptr, norm, c.eps, nullptr, n, q), "decode-GEMV");
+            return;
+        }
+        must(t12_gemv_gain_norm(&g, 1, st->y, cur, post, gain, c.eps, other, n, q), "decode-GEMV");
+        std::swap(cur, other);
+    };
+    for (const Run& r : st->runs) {
+        const Layer& L = *r.layer;
+        project(seg_of(L.w_in, st->in, L.c.in_ld()), L.norm1, L.gain1);
+        mixer(st, r, 1, 0, position, q);
+        region_linear(L.w_out, st->y, n, st->mix, L.c.out_cols(), 1, false, q);
+        waits = true;
+        post = L.gain1b;
+        if (!L.c.ff) continue;
+        const T12Glu unit = unit_of(L.c);
+        T12Segment g = seg_of(L.gate, nullptr, L.c.ff), u = seg_of(L.up, nullptr, L.c.ff);
+        must(t12_gemv_glu_gain_norm(&g, &u, &unit, st->y, cur, post, L.gain2, c.eps, other, n, st->act, q), "gate|up decode-GEMV");
+        std::swap(cur, other);
+        region_linear(L.down, st->y, n, st->act, L.c.ff, 1, false, q);
+        post = L.gain2b;
+    }
+    T12Segment g = seg_of(s->model->output_proj, s->logits, c.vocab);
+    if (c.vocab >= 8192) {      // thousands of workgroups would each rebuild the normed input: one small kernel does it once
+        const Layer& L = *st->runs.back().layer;
+        must(t12_post_norm_add(st->y, nullptr, cur, L.c.ff ? L.norm2b : L.norm1b, s->model->output_norm, c.eps, other, st->h, 0, n, 1, q), "norms");
+        must(t12_gemv(&g, 1, st->h, n, q), "head decode-GEMV");
+    } else {
+        project(g, s->model->output_norm, d.final_gain);
+    }
+}
+
 void pass(InferenceState* s, int R, int run, int max_position, const LogitsRequest& lr)
 {
     State* st = state_of(s);
+    if (!run && st->fused_b1) {
+        pass_b1_fused(s, max_position);
+        return;
+    }
     const Data& d = *data_of(s->model);
     const Config& c = d.config;
     const int n = c.width;

@@ -44,6 +44,7 @@ struct GemvParams {
     int out_ld;                            // elements between output rows (fp32 outputs and out_bf16)
     float act_a, act_b;                    // EPI launches: the constants of the unary function
     T12Glu glu = t12_silu_glu();           // SwiGLU mode: the unit
+    float gain_post, gain;                 // NORM 3: gain of the norm nx goes through, gain of the norm of the sum
 };
 
 __device__ __forceinline__ int find_segment(const GemvParams& p, int blk)
@@ -111,6 +112,8 @@ __device__ __forceinline__ float lds_act_at(const uint4* lds_act, int k)
 // workgroup rebuilds them from the fp32 residual stream while its first weight tiles are in
 // flight -- the reference's (add_)rms_norm_bf16_batch kernels (engine/kernels.hip:355-442) as a
 // prologue.  K <= 16 * NW * 64.  Workgroup 0 also stores nx + nres for the residual path.
+// NORM 3: norms with one gain for all columns, before and after the residual add: activations = bf16(rmsnorm(s) gain),
+// s = nres + rmsnorm(nx) gain_post.  (With weight vectors the prologue would read as many bytes as the workgroup's weights.)
 // EPI (T12_ACT_*): the unary function applied to every sum of a single-segment launch -- xIELU stored as bf16 to
 // p.out_bf16[m] (the front half of a feed-forward without a gate), the soft cap in place of the plain fp32 store.
 // MOE: one activation row per blockIdx.y, multiplied with the tensors of the expert slot_expert[blockIdx.y] names --
@@ -162,7 +165,7 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
     }
 
     // NORM: the same for the fp32 residual stream, its addend and the norm weights (8 columns per piece, 2 pieces per thread)
-    float4 npre[NORM ? 2 : 1][2], rpre[NORM == 2 ? 2 : 1][2], wpre[NORM ? 2 : 1][2];
+    float4 npre[NORM ? 2 : 1][2], rpre[NORM >= 2 ? 2 : 1][2], wpre[NORM ? 2 : 1][2];
     if (NORM != 0) {
 #pragma unroll
         for (int gi = 0; gi < 2; gi++) {
@@ -170,12 +173,14 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
             if (gi == 0 || NW * 64 * 8 < K) {                        // workgroup-uniform
                 npre[gi][0] = *(const float4*)(p.nx + k);
                 npre[gi][1] = *(const float4*)(p.nx + k + 4);
-                if (NORM == 2) {
+                if (NORM >= 2) {
                     rpre[gi][0] = *(const float4*)(p.nres + k);
                     rpre[gi][1] = *(const float4*)(p.nres + k + 4);
                 }
-                wpre[gi][0] = *(const float4*)(p.nw + k);
-                wpre[gi][1] = *(const float4*)(p.nw + k + 4);
+                if (NORM != 3) {
+                    wpre[gi][0] = *(const float4*)(p.nw + k);
+                    wpre[gi][1] = *(const float4*)(p.nw + k + 4);
+                }
             }
         }
     }
@@ -237,8 +242,37 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
         }
     } else {
         __shared__ float red[NW];
+        __shared__ float4 red3[NW];
         float v[2][8];
-        float ss = 0.0f;
+        float ss = 0.0f, post = 1.0f, tot3 = 0.0f;
+        if (NORM == 3) {
+            // the sum of squares of nres + a nx is |nres|^2 + 2 a (nres . nx) + a^2 |nx|^2: both norms come out of one reduction
+            float s[3] = {0.0f, 0.0f, 0.0f};
+#pragma unroll
+            for (int gi = 0; gi < 2; gi++)
+                if ((tid + gi * NW * 64) * 8 < K) {
+#pragma unroll
+                    for (int h = 0; h < 2; h++) {
+                        const float4 y = npre[gi][h], x = rpre[gi][h];
+                        s[0] += y.x * y.x + y.y * y.y + y.z * y.z + y.w * y.w;
+                        s[1] += x.x * x.x + x.y * x.y + x.z * x.z + x.w * x.w;
+                        s[2] += x.x * y.x + x.y * y.y + x.z * y.z + x.w * y.w;
+                    }
+                }
+#pragma unroll
+            for (int q = 0; q < 3; q++) s[q] = t12_wave_sum_lane63(s[q]);
+            if (lane == 63) red3[wave] = make_float4(s[0], s[1], s[2], 0.0f);
+            __syncthreads();
+            float4 t = red3[0];
+#pragma unroll
+            for (int w = 1; w < NW; w++) {
+                t.x += red3[w].x;
+                t.y += red3[w].y;
+                t.z += red3[w].z;
+            }
+            post = p.gain_post / sqrtf(t.x / (float)K + p.eps);
+            tot3 = fmaxf(t.y + 2.0f * post * t.z + post * post * t.x, 0.0f);
+        }
 #pragma unroll
         for (int gi = 0; gi < 2; gi++) {
             const int k = (tid + gi * NW * 64) * 8;
@@ -248,7 +282,11 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
                 const float4 a = npre[gi][0], b = npre[gi][1];
                 v[gi][0] = a.x; v[gi][1] = a.y; v[gi][2] = a.z; v[gi][3] = a.w;
                 v[gi][4] = b.x; v[gi][5] = b.y; v[gi][6] = b.z; v[gi][7] = b.w;
-                if (NORM == 2) {
+                if (NORM == 3) {
+#pragma unroll
+                    for (int e = 0; e < 8; e++) v[gi][e] *= post;
+                }
+                if (NORM >= 2) {
                     const float4 c = rpre[gi][0], d = rpre[gi][1];
                     v[gi][0] += c.x; v[gi][1] += c.y; v[gi][2] += c.z; v[gi][3] += c.w;
                     v[gi][4] += d.x; v[gi][5] += d.y; v[gi][6] += d.z; v[gi][7] += d.w;
@@ -261,13 +299,16 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
                 for (int e = 0; e < 8; e++) ss += v[gi][e] * v[gi][e];
             }
         }
-        ss = t12_wave_sum(ss);
-        if (lane == 0) red[wave] = ss;
-        __syncthreads();
-        float tot = 0.0f;
+        float tot = tot3;
+        if (NORM != 3) {
+            ss = t12_wave_sum(ss);
+            if (lane == 0) red[wave] = ss;
+            __syncthreads();
+            tot = 0.0f;
 #pragma unroll
-        for (int w = 0; w < NW; w++) tot += red[w];
-        const float rn = rsqrtf(tot / (float)K + p.eps);
+            for (int w = 0; w < NW; w++) tot += red[w];
+        }
+        const float rn = NORM == 3 ? p.gain / sqrtf(tot / (float)K + p.eps) : rsqrtf(tot / (float)K + p.eps);
 #pragma unroll
         for (int gi = 0; gi < 2; gi++) {
             const int q = tid + gi * NW * 64;
@@ -275,7 +316,8 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
             if (q < nchunk * 128) {
                 uint4 y = make_uint4(0, 0, 0, 0);
                 if (k < K) {
-                    const float4 wa = wpre[gi][0], wb = wpre[gi][1];
+                    const float4 one = make_float4(1.0f, 1.0f, 1.0f, 1.0f);
+                    const float4 wa = NORM == 3 ? one : wpre[gi][0], wb = NORM == 3 ? one : wpre[gi][1];
                     y.x = t12_f32_to_bf16(v[gi][0] * rn * wa.x) | ((uint32_t)t12_f32_to_bf16(v[gi][1] * rn * wa.y) << 16);
                     y.y = t12_f32_to_bf16(v[gi][2] * rn * wa.z) | ((uint32_t)t12_f32_to_bf16(v[gi][3] * rn * wa.w) << 16);
                     y.z = t12_f32_to_bf16(v[gi][4] * rn * wb.x) | ((uint32_t)t12_f32_to_bf16(v[gi][5] * rn * wb.y) << 16);
@@ -702,6 +744,60 @@ int t12_gemv_act(const T12Segment* seg, const void* act_bf16, const float* x, co
     hipStream_t st = (hipStream_t)stream;
     if (act_bf16) return act->kind == T12_ACT_XIELU ? launch_act<0, T12_ACT_XIELU>(p, st) : launch_act<0, T12_ACT_SOFTCAP>(p, st);
     return act->kind == T12_ACT_XIELU ? launch_act<1, T12_ACT_XIELU>(p, st) : launch_act<1, T12_ACT_SOFTCAP>(p, st);
+}
+
+// y_s = W_s . bf16(rmsnorm(sum) gain), sum = residual + rmsnorm(x) gain_post, both norms in the kernel's prologue.
+int t12_gemv_gain_norm(const T12Segment* segs, int nseg, const float* x, const float* residual, float gain_post, float gain, float eps,
+                       float* hidden_out, int K, void* stream)
+{
+    T12_REQUIRE(residual, "t12_gemv_gain_norm: residual is null");
+    int rc = validate(segs, nseg, x, K, true);
+    if (rc) return rc;
+    rc = check_norm_operands("t12_gemv_gain_norm", segs, nseg, x, residual, x, hidden_out, K);
+    if (rc) return rc;
+    GemvParams p;
+    for (int i = 0; i < nseg; i++) p.seg[i] = segs[i];
+    p.nseg = nseg;
+    p.K = K;
+    p.act = nullptr;
+    p.out_bf16 = nullptr;
+    p.add = nullptr;
+    p.nx = x;
+    p.nres = residual;
+    p.hidden_out = hidden_out;
+    p.eps = eps;
+    p.gain_post = gain_post;
+    p.gain = gain;
+    return launch_plain_norm<3>(p, segs, nseg, (hipStream_t)stream);
+}
+
+// The same for a gate|up pair with a gated linear unit in the epilogue.
+int t12_gemv_glu_gain_norm(const T12Segment* gate, const T12Segment* up, const T12Glu* glu, const float* x, const float* residual,
+                           float gain_post, float gain, float eps, float* hidden_out, int K, void* out_bf16, void* stream)
+{
+    T12_REQUIRE(gate && up && glu && residual && out_bf16, "t12_gemv_glu_gain_norm: null operand");
+    T12Segment two[2] = {*gate, *up};
+    int rc = validate(two, 2, x, K, false);
+    if (rc) return rc;
+    T12_REQUIRE(gate->M == up->M, "t12_gemv_glu_gain_norm: gate has %d rows, up has %d", gate->M, up->M);
+    rc = check_norm_operands("t12_gemv_glu_gain_norm", two, 2, x, residual, x, hidden_out, K);
+    if (rc) return rc;
+    GemvParams p;
+    p.glu = *glu;
+    p.seg[0] = two[0];
+    p.seg[1] = two[1];
+    p.nseg = 2;
+    p.K = K;
+    p.act = nullptr;
+    p.out_bf16 = (uint16_t*)out_bf16;
+    p.add = nullptr;
+    p.nx = x;
+    p.nres = residual;
+    p.hidden_out = hidden_out;
+    p.eps = eps;
+    p.gain_post = gain_post;
+    p.gain = gain;
+    return launch_swiglu<3>(p, (hipStream_t)stream);
 }
 
 // One activation row per slot, each multiplied with the tensors of the expert the routing gave the slot (a device
