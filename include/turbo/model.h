@@ -97,8 +97,8 @@ Model* load_model(const std::string& model_path, int device_id = 0);
 // row and ascending within it.  false + the first finding in err.
 //
 // Other families are told apart by the directory (load_model asks each in turn): one with a config.json whose
-// "architecture" names a family of this build -- "Gamilorn": config.json + model.safetensors, packed on the GPU while
-// loading, or the split-12 directory save_model writes for it -- is checked and loaded by that family.
+// "architecture" names a family of this build -- "Gamilorn", "Davasun": config.json + model.safetensors, packed on the GPU
+// while loading, or the split-12 directory save_model writes for it -- is checked and loaded by that family.
 bool check_model_dir(const std::string& model_path, std::string& err);
 void free_model(Model* model);
 const char* model_family(const Model* model);    // "llama", "gamilorn", "davasun"

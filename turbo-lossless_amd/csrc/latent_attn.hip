@@ -5,9 +5,9 @@
 // the value projection at the end.  So attention runs over one shared "head" of rank + rot_dim channels whose values are the
 // first rank of them, and a token's cache is that one row.
 //
-// A step is three launches: the key projection of the queries (beside it, in workgroups of their own, the cache store and the
-// rotations; a launch of its own in prompt passes), attention, the value projection with the gate.  All three run on the matrix cores for the sizes that have
-// instances; 32-bit states and other sizes take the general forms.
+// A pass is the cache store with the rotations, the key projection of the queries, attention, the value projection with the gate;
+// with few rows the store runs beside the key projection, in workgroups of its own.  All of them run on the matrix cores for the
+// sizes that have instances; 32-bit states and other sizes take the general forms.
 
 #include <algorithm>
 #include <mutex>
