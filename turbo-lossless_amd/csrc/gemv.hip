@@ -226,6 +226,13 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
         __builtin_amdgcn_sched_barrier(0);   // issue in ring order: waits can then be partial
     }
 
+    // What the last instructions need of the launch's arguments, asked for now: a scalar load at the end would be waited for alone.
+    T12Glu glu = p.glu;
+    uint16_t* out16 = p.out_bf16;
+    float act_a = p.act_a, act_b = p.act_b;
+    if (SWIGLU) asm volatile("" : "+s"(glu.limit), "+s"(glu.slope), "+s"(glu.offset), "+s"(out16));
+    if (EPI != T12_ACT_NONE) asm volatile("" : "+s"(act_a), "+s"(act_b), "+s"(out16));
+
     if (NORM == 0) {
 #pragma unroll
         for (int u = 0; u < SU; u++) {
@@ -393,15 +400,15 @@ __global__ __launch_bounds__(NW * 64, MINB) void gemv_stream_kernel(const GemvPa
                      lds_act_at(lds_act, SEG(r).cols[q]);
             tot[r] = t12_wave_sum_lane63(v);
             if (!SWIGLU && lane == 63) {
-                if (EPI == T12_ACT_XIELU) p.out_bf16[row0 + r] = t12_f32_to_bf16(t12_apply_act<EPI>(tot[r], p.act_a, p.act_b));
-                else if (EPI != T12_ACT_NONE) sg.out[row0 + r] = t12_apply_act<EPI>(tot[r], p.act_a, p.act_b);
+                if (EPI == T12_ACT_XIELU) out16[row0 + r] = t12_f32_to_bf16(t12_apply_act<EPI>(tot[r], act_a, act_b));
+                else if (EPI != T12_ACT_NONE) sg.out[row0 + r] = t12_apply_act<EPI>(tot[r], act_a, act_b);
                 else if (MOE) sg.out[(size_t)blockIdx.y * p.out_ld + row0 + r] = tot[r];
                 else sg.out[row0 + r] = p.add ? tot[r] + p.add[row0 + r] : tot[r];
             }
         }
     }
     if (SWIGLU && lane == 63) {
-        (MOE ? p.out_bf16 + (size_t)blockIdx.y * p.out_ld : p.out_bf16)[row0] = t12_f32_to_bf16(t12_apply_glu(tot[0], tot[R - 1], p.glu));
+        (MOE ? out16 + (size_t)blockIdx.y * p.out_ld : out16)[row0] = t12_f32_to_bf16(t12_apply_glu(tot[0], tot[R - 1], glu));
     }
 #undef SEG
 #undef ROW

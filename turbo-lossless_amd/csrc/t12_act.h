@@ -16,8 +16,8 @@ __device__ __forceinline__ float t12_sigmoid(float x) { return 1.0f / (1.0f + ex
 // Gated linear unit of a (gate, up) pair of sums.
 __device__ __forceinline__ float t12_apply_glu(float g, float u, const T12Glu& p)
 {
-    g = g > p.limit ? p.limit : g;
-    u = u > p.limit ? p.limit : u < -p.limit ? -p.limit : u;
+    g = fminf(g, p.limit);
+    u = __builtin_amdgcn_fmed3f(u, -p.limit, p.limit);
     return g / (1.0f + expf(-p.slope * g)) * (u + p.offset);
 }
 
